@@ -6,8 +6,11 @@
 //                            mixture's  sum_j wts[t, j] * rows[inv[t, j]]  (+ [sigmoid(gate[t]) *] shared[t])
 //                   xs'[t] = sum_s mix[s, t] xs[s] + a_out[t] y          (all streams from the old ones)
 //                   u      = sum_t a_in[t] xs'[t];  z = u / sqrt(mean(u^2) + eps) * w
-//                 either half may be absent; with `rows` only those tokens are opened (the rows whose
+//                 y may first be set to unit RMS times a weight (post_w) or be scaled coordinate by
+//                 coordinate (y_scale); without a norm weight the opened sum u itself is z.
+//                 Either half may be absent; with `rows` only those tokens are opened (the rows whose
 //                 logits are wanted).  S = 1 with unit coefficients is the plain residual.
+//   embed_norm    x[t] = table[ids[t]] set to unit RMS times a weight, as fp32
 //   tanh_cap      x <- cap * tanh(x / cap)
 //
 // One workgroup per token; every sum runs in a fixed order, so a token's result does not depend
@@ -55,6 +58,8 @@ struct HyperArgs {
   void* act;
   float* z32;
   const int* rows;
+  const float* y_scale;  // [W] or null
+  const float* post_w;   // [W] or null: y <- y / sqrt(mean(y^2) + eps) * post_w
 };
 
 // four consecutive coordinates per thread (W % 4 == 0): 16-byte loads of the fp32 streams
@@ -79,21 +84,59 @@ __device__ __forceinline__ void st4<bf16_t>(bf16_t* p, float4 v) {
   w.y = pk::pack2(v.z, v.w);
   *reinterpret_cast<uint2*>(p) = w;
 }
+__device__ __forceinline__ float4 mul4(float4 a, float4 b) { return float4{a.x * b.x, a.y * b.y, a.z * b.z, a.w * b.w}; }
 __device__ __forceinline__ float4 fma4(float c, float4 a, float4 b) {
   return float4{c * a.x + b.x, c * a.y + b.y, c * a.z + b.z, c * a.w + b.w};
 }
 
+// the sublayer output at coordinates i .. i + 3 / at coordinate i of token src
+template <typename T, typename Y>
+__device__ __forceinline__ float4 sublayer_out4(const HyperArgs& a, int64_t src, int i, float gate) {
+  const Y* y = static_cast<const Y*>(a.y);
+  const T* y2 = static_cast<const T*>(a.y2);
+  float4 yv = float4{0.f, 0.f, 0.f, 0.f};
+  if (a.inv) {
+    for (int j = 0; j < a.top; ++j) {
+      const int row = a.inv[src * a.top + j];
+      if (row >= 0) yv = fma4(a.wts[src * a.top + j], ld4<Y>(y + static_cast<int64_t>(row) * a.W + i), yv);
+    }
+  } else if (y) {
+    yv = ld4<Y>(y + src * a.W + i);
+    for (int sl = 1; sl < a.nslab; ++sl) yv = fma4(1.f, ld4<Y>(y + sl * a.slab_stride + src * a.W + i), yv);
+  }
+  if (y2) yv = fma4(gate, ld4<T>(y2 + src * a.W + i), yv);
+  return yv;
+}
+template <typename T, typename Y>
+__device__ __forceinline__ float sublayer_out(const HyperArgs& a, int64_t src, int i, float gate) {
+  const Y* y = static_cast<const Y*>(a.y);
+  const T* y2 = static_cast<const T*>(a.y2);
+  float yv = 0.f;
+  if (a.inv) {
+    for (int j = 0; j < a.top; ++j) {
+      const int row = a.inv[src * a.top + j];
+      if (row >= 0) yv += a.wts[src * a.top + j] * ld<Y>(y + static_cast<int64_t>(row) * a.W + i);
+    }
+  } else if (y) {
+    yv = ld<Y>(y + src * a.W + i);
+    for (int sl = 1; sl < a.nslab; ++sl) yv += ld<Y>(y + sl * a.slab_stride + src * a.W + i);
+  }
+  if (y2) yv += gate * ld<T>(y2 + src * a.W + i);
+  return yv;
+}
+
 // VEC >= 4 (= 4 * groups per thread): W % 4 == 0, every thread owns up to VEC / 4 groups of four
 // consecutive coordinates and keeps the opened sum in registers between the two passes; VEC = 1: any
-// W, one coordinate at a time, the opened sum in LDS
-template <typename T, typename Y, int VEC>
+// W, one coordinate at a time, the opened sum in LDS.  POST: the sublayer output is normed first.
+// NS: the most streams this form handles (1 or kMaxStreams).
+template <typename T, typename Y, int VEC, bool POST, int NS>
 __global__ void __launch_bounds__(1024) hyper_step_kernel(HyperArgs a) {
   constexpr int NG = VEC >= 4 ? VEC / 4 : 1;
   __shared__ float red[16];
   __shared__ float cf[kMaxStreams * kMaxStreams + 2 * kMaxStreams];
   extern __shared__ __attribute__((aligned(16))) float vbuf[];  // [W] the opened sum u, kept between the two passes
   const int r = blockIdx.x;
-  const int S = a.S, W = a.W;
+  const int S = NS == 1 ? 1 : a.S, W = a.W;
   const int64_t src = a.rows ? a.rows[r] : r;
   float* x = a.xs + src * S * W;
   const bool close = a.mix != nullptr, open = a.a_in != nullptr;
@@ -106,35 +149,52 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(HyperArgs a) {
     if (open) c_in[threadIdx.x] = a.a_in[threadIdx.x];
   }
   __syncthreads();
-  const Y* y = static_cast<const Y*>(a.y);
-  const T* y2 = static_cast<const T*>(a.y2);
-  const float gate = y2 ? (a.g2 ? sigmoidf(a.g2[src * a.g2_stride]) : 1.f) : 0.f;
+  const float gate = a.y2 ? (a.g2 ? sigmoidf(a.g2[src * a.g2_stride]) : 1.f) : 0.f;
   float ss = 0.f;
   float4 ur[NG];
+  float ky = 1.f;
+  if (POST) {
+    float sy = 0.f;
+    if (VEC >= 4) {
+#pragma unroll
+      for (int it = 0; it < NG; ++it) {
+        const int i = 4 * (threadIdx.x + it * blockDim.x);
+        if (i >= W) break;
+        const float4 v = sublayer_out4<T, Y>(a, src, i, gate);
+        ur[it] = v;
+        sy += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+      }
+    } else {
+      for (int i = threadIdx.x; i < W; i += blockDim.x) {
+        const float v = sublayer_out<T, Y>(a, src, i, gate);
+        vbuf[i] = v;
+        sy += v * v;
+      }
+    }
+    ky = 1.f / sqrtf(pk::block_sum(sy, red) / static_cast<float>(W) + a.eps);
+    __syncthreads();
+  }
   if (VEC >= 4) {
 #pragma unroll
     for (int it = 0; it < NG; ++it) {
       const int i = 4 * (threadIdx.x + it * blockDim.x);
       if (i >= W) break;
-      float4 xv[kMaxStreams];
+      float4 xv[NS];
 #pragma unroll
-      for (int s = 0; s < kMaxStreams; ++s)
+      for (int s = 0; s < NS; ++s)
         if (s < S) xv[s] = ld4<float>(x + s * W + i);
       if (close) {
-        float4 yv = float4{0.f, 0.f, 0.f, 0.f};
-        if (a.inv) {
-          for (int j = 0; j < a.top; ++j) {
-            const int row = a.inv[src * a.top + j];
-            if (row >= 0) yv = fma4(a.wts[src * a.top + j], ld4<Y>(y + static_cast<int64_t>(row) * W + i), yv);
-          }
-        } else if (y) {
-          yv = ld4<Y>(y + src * W + i);
-          for (int sl = 1; sl < a.nslab; ++sl) yv = fma4(1.f, ld4<Y>(y + sl * a.slab_stride + src * W + i), yv);
+        float4 yv;
+        if (POST) {
+          const float4 v = ur[it];
+          yv = mul4(float4{v.x * ky, v.y * ky, v.z * ky, v.w * ky}, ld4<float>(a.post_w + i));
+        } else {
+          yv = sublayer_out4<T, Y>(a, src, i, gate);
         }
-        if (y2) yv = fma4(gate, ld4<T>(y2 + src * W + i), yv);
-        float4 nv[kMaxStreams];
+        if (a.y_scale) yv = mul4(yv, ld4<float>(a.y_scale + i));
+        float4 nv[NS];
 #pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t) {
+        for (int t = 0; t < NS; ++t) {
           if (t < S) {
             float4 acc = float4{0.f, 0.f, 0.f, 0.f};
             for (int s = 0; s < S; ++s) acc = fma4(c_mix[s * S + t], xv[s], acc);
@@ -143,13 +203,13 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(HyperArgs a) {
           }
         }
 #pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t)
+        for (int t = 0; t < NS; ++t)
           if (t < S) xv[t] = nv[t];
       }
       if (open) {
         float4 u = float4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t)
+        for (int t = 0; t < NS; ++t)
           if (t < S) u = fma4(c_in[t], xv[t], u);
         ur[it] = u;
         ss += (u.x * u.x + u.y * u.y) + (u.z * u.z + u.w * u.w);
@@ -157,24 +217,15 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(HyperArgs a) {
     }
   } else {
     for (int i = threadIdx.x; i < W; i += blockDim.x) {
-      float xv[kMaxStreams];
+      float xv[NS];
 #pragma unroll
-      for (int s = 0; s < kMaxStreams; ++s) xv[s] = s < S ? x[s * W + i] : 0.f;
+      for (int s = 0; s < NS; ++s) xv[s] = s < S ? x[s * W + i] : 0.f;
       if (close) {
-        float yv = 0.f;
-        if (a.inv) {
-          for (int j = 0; j < a.top; ++j) {
-            const int row = a.inv[src * a.top + j];
-            if (row >= 0) yv += a.wts[src * a.top + j] * ld<Y>(y + static_cast<int64_t>(row) * W + i);
-          }
-        } else if (y) {
-          yv = ld<Y>(y + src * W + i);
-          for (int sl = 1; sl < a.nslab; ++sl) yv += ld<Y>(y + sl * a.slab_stride + src * W + i);
-        }
-        if (y2) yv += gate * ld<T>(y2 + src * W + i);
-        float nv[kMaxStreams];
+        float yv = POST ? vbuf[i] * ky * a.post_w[i] : sublayer_out<T, Y>(a, src, i, gate);
+        if (a.y_scale) yv *= a.y_scale[i];
+        float nv[NS];
 #pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t) {
+        for (int t = 0; t < NS; ++t) {
           if (t < S) {
             float acc = 0.f;
             for (int s = 0; s < S; ++s) acc += c_mix[s * S + t] * xv[s];
@@ -183,12 +234,12 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(HyperArgs a) {
           }
         }
 #pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t) xv[t] = t < S ? nv[t] : 0.f;
+        for (int t = 0; t < NS; ++t) xv[t] = t < S ? nv[t] : 0.f;
       }
       if (open) {
         float u = 0.f;
 #pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t)
+        for (int t = 0; t < NS; ++t)
           if (t < S) u += c_in[t] * xv[t];
         vbuf[i] = u;
         ss += u * u;
@@ -196,26 +247,48 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(HyperArgs a) {
     }
   }
   if (!open) return;
-  ss = pk::block_sum(ss, red);
-  const float k = 1.f / sqrtf(ss / static_cast<float>(W) + a.eps);
+  float k = 1.f;
+  if (a.norm_w) {
+    ss = pk::block_sum(ss, red);
+    k = 1.f / sqrtf(ss / static_cast<float>(W) + a.eps);
+  }
   T* act = static_cast<T*>(a.act);
   if (VEC >= 4) {
 #pragma unroll
     for (int it = 0; it < NG; ++it) {
       const int i = 4 * (threadIdx.x + it * blockDim.x);
       if (i >= W) break;
-      const float4 u = ur[it], g = ld4<float>(a.norm_w + i);
+      const float4 u = ur[it], g = a.norm_w ? ld4<float>(a.norm_w + i) : float4{1.f, 1.f, 1.f, 1.f};
       const float4 z = float4{u.x * k * g.x, u.y * k * g.y, u.z * k * g.z, u.w * k * g.w};
       if (act) st4<T>(act + static_cast<int64_t>(r) * W + i, z);
       if (a.z32) st4<float>(a.z32 + static_cast<int64_t>(r) * W + i, z);
     }
   } else {
     for (int i = threadIdx.x; i < W; i += blockDim.x) {
-      const float z = vbuf[i] * k * a.norm_w[i];
+      const float z = a.norm_w ? vbuf[i] * k * a.norm_w[i] : vbuf[i];
       if (act) st<T>(act + static_cast<int64_t>(r) * W + i, z);
       if (a.z32) a.z32[static_cast<int64_t>(r) * W + i] = z;
     }
   }
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) embed_norm_kernel(float* __restrict__ x, const T* __restrict__ table,
+                                                         const int* __restrict__ ids, const float* __restrict__ w, int W,
+                                                         int vocab, float eps) {
+  __shared__ float red[16];
+  const int t = blockIdx.x;
+  int id = ids[t];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  const T* src = table + static_cast<int64_t>(id) * W;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float v = ld<T>(src + i);
+    ss += v * v;
+  }
+  ss = pk::block_sum(ss, red);
+  const float k = 1.f / sqrtf(ss / static_cast<float>(W) + eps);
+  for (int i = threadIdx.x; i < W; i += blockDim.x) x[static_cast<int64_t>(t) * W + i] = ld<T>(src + i) * k * w[i];
 }
 
 __global__ void __launch_bounds__(256) tanh_cap_kernel(float* __restrict__ x, int64_t n, float cap) {
@@ -234,25 +307,41 @@ PK_EXPORT int pkm_spread_rows(void* xs, const void* table, const void* ids, int 
   return PK_CHECK_LAUNCH();
 }
 
+// x [T, W] fp32 <- unit-RMS rows of the table times w [W]
+PK_EXPORT int pkm_embed_norm(void* x, const void* table, const void* ids, const void* w, int T, int W, int vocab, float eps,
+                             int dt, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (W < 1 || vocab < 1) return -1;
+  PKM_DISPATCH(dt, E, embed_norm_kernel<E><<<T, 256, 0, stream>>>(static_cast<float*>(x), static_cast<const E*>(table),
+                                                                   static_cast<const int*>(ids), static_cast<const float*>(w),
+                                                                   W, vocab, eps));
+  return PK_CHECK_LAUNCH();
+}
+
 // xs [tokens, S, W] fp32, updated in place when mix / a_out are given (then y, or inv / wts / y rows,
 // is the sublayer output; y_dt its element type, -1: none).  y2 / g2: a second row per token in the
 // activation type and its pre-sigmoid gate (fp32, element stride g2_stride; null: the row is added as it is).  a_in / norm_w: open.
-// rows: R token indices to open (no close).  act (element type act_dt) and z32 may each be null.
+// norm_w null with a_in: the opened sum as it is.  y_scale, post_w [W] fp32 or null: y scaled per coordinate /
+// set to unit RMS times post_w (S = 1 only) before it is folded in.  rows: R token indices to open (no close).  act (element type act_dt) and z32 may each be null.
 PK_EXPORT int pkm_hyper_step(void* xs, int R, int S, int W, const void* y, int y_dt, int nslab, const void* inv, int top,
                              const void* wts, const void* y2, int y2_dt, const void* g2, long long g2_stride,
                              const void* mix, const void* a_out, const void* a_in, const void* norm_w, float eps,
-                             void* act, int act_dt, void* z32, const void* rows, hipStream_t stream) {
+                             void* act, int act_dt, void* z32, const void* rows, const void* y_scale,
+                             const void* post_w, hipStream_t stream) {
   if (R <= 0) return 0;
   if (S < 1 || S > kMaxStreams || W > 16384 || nslab < 1) return -1;
-  if ((mix == nullptr) != (a_out == nullptr) || (a_in == nullptr) != (norm_w == nullptr)) return -1;
+  if ((mix == nullptr) != (a_out == nullptr) || (norm_w != nullptr && a_in == nullptr)) return -1;
+  if ((y_scale || post_w) && (!mix || !y)) return -1;
+  if (post_w && S != 1) return -1;
   if (rows && mix) return -1;
   if (inv && (!y || !wts || top < 1 || nslab > 1)) return -1;
   if (y2 && y2_dt != act_dt) return -1;
   HyperArgs a{static_cast<float*>(xs), S, W, y, nslab, static_cast<int64_t>(R) * W, static_cast<const int*>(inv), top,
               static_cast<const float*>(wts), y2, static_cast<const float*>(g2), g2_stride,
               static_cast<const float*>(mix), static_cast<const float*>(a_out), static_cast<const float*>(a_in),
-              static_cast<const float*>(norm_w), eps, act, static_cast<float*>(z32), static_cast<const int*>(rows)};
-  const size_t lds = a_in ? static_cast<size_t>(W) * sizeof(float) : 0;
+              static_cast<const float*>(norm_w), eps, act, static_cast<float*>(z32), static_cast<const int*>(rows),
+              static_cast<const float*>(y_scale), static_cast<const float*>(post_w)};
+  const size_t lds = (a_in || post_w) ? static_cast<size_t>(W) * sizeof(float) : 0;
   if (y_dt != kF32 && y_dt != kBF16 && y != nullptr) return -2;
   const bool y32 = y == nullptr || y_dt == kF32;
   if (W % 4 == 0) {  // up to 256 threads, each with 1, 2, 4 or 8 groups of four coordinates
@@ -264,7 +353,14 @@ PK_EXPORT int pkm_hyper_step(void* xs, int R, int S, int W, const void* y, int y
     int threads = (want + 63) / 64 * 64;
     threads = threads > 1024 ? 1024 : threads;
     const int per = (groups + threads - 1) / threads;
-#define PKM_HS(YT, VEC) PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, YT, VEC><<<R, threads, 0, stream>>>(a))
+#define PKM_HS(YT, VEC)                                                                             \
+  if (post_w) {                                                                                                \
+    PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, YT, VEC, true, 1><<<R, threads, 0, stream>>>(a));             \
+  } else if (S == 1) {                                                                                         \
+    PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, YT, VEC, false, 1><<<R, threads, 0, stream>>>(a));            \
+  } else {                                                                                                     \
+    PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, YT, VEC, false, kMaxStreams><<<R, threads, 0, stream>>>(a));  \
+  }
 #define PKM_HS_Y(VEC)   \
   if (y32) {            \
     PKM_HS(float, VEC); \
@@ -285,12 +381,19 @@ PK_EXPORT int pkm_hyper_step(void* xs, int R, int S, int W, const void* y, int y
 #undef PKM_HS_Y
 #undef PKM_HS
   } else {
+#define PKM_HS1(YT)                                                                               \
+  if (post_w) {                                                                                             \
+    PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, YT, 1, true, 1><<<R, threads, lds, stream>>>(a));            \
+  } else {                                                                                                  \
+    PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, YT, 1, false, kMaxStreams><<<R, threads, lds, stream>>>(a)); \
+  }
     const int threads = W >= 4096 ? 1024 : (W >= 1024 ? 512 : 256);
     if (y32) {
-      PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, float, 1><<<R, threads, lds, stream>>>(a));
+      PKM_HS1(float)
     } else {
-      PKM_DISPATCH(act_dt, E, hyper_step_kernel<E, bf16_t, 1><<<R, threads, lds, stream>>>(a));
+      PKM_HS1(bf16_t)
     }
+#undef PKM_HS1
   }
   return PK_CHECK_LAUNCH();
 }

@@ -2,6 +2,8 @@
 //
 //     S_t = decay_h * S_{t-1} + k_t v_t^T        o_t = S_t^T q_t        q, k, v = silu(projections)
 //
+// Retention is the same recurrence on plain projections (no SiLU): q and k turn by the token's
+// position in fp32 (pair (i, i + pairs), (cos, sin) table rows) and k is multiplied by k_scale.
 // The state S [D, V] of a (sequence, head) is fp32 and lives in the sequence's state slot between
 // steps.  One workgroup owns 16 value columns of one (sequence, head): thread (dg, vc) keeps rows
 // dg, dg + 16, ... of column vc in registers and walks the portion's tokens in order; q, k, v of up to
@@ -18,13 +20,34 @@ namespace {
 constexpr int kMaxChunk = 32;  // tokens staged per group (fewer when a head is wide)
 constexpr int kCols = 16;   // value columns per workgroup
 
+// what happens to a projection on its way into the recurrence
+struct HeadIn {
+  const float* table;    // [rows, pairs, 2] fp32 (cos, sin) or null
+  int pairs, rows;
+  const int* positions;
+  float k_scale;
+};
+
 __device__ __forceinline__ float siluf(float z) { return z / (1.f + expf(-z)); }
 
-template <typename T, int ND>
+// coordinate d of a head's projection row `src`, turned by token t's position
+template <typename T>
+__device__ __forceinline__ float turned(const T* src, int d, int64_t t, const HeadIn& in) {
+  const float x = ld<T>(src + d);
+  if (in.table == nullptr || d >= 2 * in.pairs) return x;
+  const bool first = d < in.pairs;
+  const int i = first ? d : d - in.pairs;
+  const float y = ld<T>(src + (first ? d + in.pairs : i));
+  const int pos = in.positions[t];
+  const float* cs = in.table + (static_cast<int64_t>(pos < 0 ? 0 : min(pos, in.rows - 1)) * in.pairs + i) * 2;
+  return first ? x * cs[0] - y * cs[1] : x * cs[0] + y * cs[1];
+}
+
+template <typename T, int ND, bool RET>
 __global__ void __launch_bounds__(256)
 lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t stride, float* __restrict__ state,
                  const float* __restrict__ decay, const int* __restrict__ cu_q, const int* __restrict__ positions,
-                 const int* __restrict__ slots, int H, int D, int V, int kChunk) {
+                 const int* __restrict__ slots, int H, int D, int V, int kChunk, HeadIn in) {
   extern __shared__ float smem[];
   float* qs = smem;                 // [kChunk][D]
   float* ks = qs + kChunk * D;      // [kChunk][D]
@@ -53,12 +76,13 @@ lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t str
     for (int e = tid; e < nt * D; e += 256) {
       const int t = e / D, d = e - t * D;
       const T* row = qkv + static_cast<int64_t>(t0 + t) * stride;
-      qs[e] = siluf(ld<T>(row + qo + d));
-      ks[e] = siluf(ld<T>(row + ko + d));
+      qs[e] = RET ? turned(row + qo, d, t0 + t, in) : siluf(ld<T>(row + qo + d));
+      ks[e] = RET ? turned(row + ko, d, t0 + t, in) * in.k_scale : siluf(ld<T>(row + ko + d));
     }
     for (int e = tid; e < nt * kCols; e += 256) {
       const int t = e / kCols, c = e - t * kCols;
-      vs[e] = v0 + c < V ? siluf(ld<T>(qkv + static_cast<int64_t>(t0 + t) * stride + vo + c)) : 0.f;
+      const float v = v0 + c < V ? ld<T>(qkv + static_cast<int64_t>(t0 + t) * stride + vo + c) : 0.f;
+      vs[e] = RET ? v : siluf(v);
     }
     __syncthreads();
     for (int t = 0; t < nt; ++t) {
@@ -99,11 +123,11 @@ lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t str
 constexpr int kWideChunk = 16;
 constexpr int kWideCols = 64;
 
-template <typename T, int NR, int NW>
+template <typename T, int NR, int NW, bool RET>
 __global__ void __launch_bounds__(64 * NW)
 lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t stride, float* __restrict__ state,
                       const float* __restrict__ decay, const int* __restrict__ cu_q, const int* __restrict__ positions,
-                      const int* __restrict__ slots, int H, int D, int V) {
+                      const int* __restrict__ slots, int H, int D, int V, HeadIn in) {
   constexpr int DP = NW * NR;  // padded key width: rows past D hold zeros
   constexpr int NT = 64 * NW;
   constexpr int QK_IT = (kWideChunk * DP + NT - 1) / NT, V_IT = (kWideChunk * kWideCols + NT - 1) / NT;
@@ -137,14 +161,19 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
       const int e = tid + NT * i, t = e / DP, d = e - t * DP;
       const bool ok = t < nt && d < D;
       const T* row = qkv + static_cast<int64_t>(t0 + (ok ? t : 0)) * stride;
-      rq[i] = ok ? ld<T>(row + qo + d) : -INFINITY;
-      rk[i] = ok ? ld<T>(row + ko + d) : -INFINITY;
+      if (RET) {
+        rq[i] = ok ? turned(row + qo, d, t0 + t, in) : 0.f;
+        rk[i] = ok ? turned(row + ko, d, t0 + t, in) * in.k_scale : 0.f;
+      } else {
+        rq[i] = ok ? ld<T>(row + qo + d) : -INFINITY;
+        rk[i] = ok ? ld<T>(row + ko + d) : -INFINITY;
+      }
     }
 #pragma unroll
     for (int i = 0; i < V_IT; ++i) {
       const int e = tid + NT * i, t = e / kWideCols, c = e - t * kWideCols;
       const bool ok = t < nt && v0 + c < V;
-      rv[i] = ok ? ld<T>(qkv + static_cast<int64_t>(t0 + (ok ? t : 0)) * stride + vo + c) : -INFINITY;
+      rv[i] = ok ? ld<T>(qkv + static_cast<int64_t>(t0 + (ok ? t : 0)) * stride + vo + c) : (RET ? 0.f : -INFINITY);
     }
   };
   fetch(a);
@@ -154,14 +183,14 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
     for (int i = 0; i < QK_IT; ++i) {
       const int e = tid + NT * i;
       if (e < kWideChunk * DP) {
-        (&qs[0][0])[e] = rq[i] == -INFINITY ? 0.f : siluf(rq[i]);
-        (&ks[0][0])[e] = rk[i] == -INFINITY ? 0.f : siluf(rk[i]);
+        (&qs[0][0])[e] = RET ? rq[i] : (rq[i] == -INFINITY ? 0.f : siluf(rq[i]));
+        (&ks[0][0])[e] = RET ? rk[i] : (rk[i] == -INFINITY ? 0.f : siluf(rk[i]));
       }
     }
 #pragma unroll
     for (int i = 0; i < V_IT; ++i) {
       const int e = tid + NT * i;
-      if (e < kWideChunk * kWideCols) (&vs[0][0])[e] = rv[i] == -INFINITY ? 0.f : siluf(rv[i]);
+      if (e < kWideChunk * kWideCols) (&vs[0][0])[e] = RET ? rv[i] : (rv[i] == -INFINITY ? 0.f : siluf(rv[i]));
     }
     __syncthreads();
     if (t0 + kWideChunk < b) fetch(t0 + kWideChunk);  // in flight while this group is computed
@@ -220,22 +249,21 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
 
 }  // namespace
 
-// out [T, H, V] fp32; qkv [T, H*D | H*D | H*V] pre-activation (row stride `stride` elements);
-// state [slots, H, D, V] fp32; sequences 0..n_seqs-1 own tokens cu_q[s]..cu_q[s+1]-1.
-PK_EXPORT int pkm_lightning_attention(void* out, const void* qkv, long long stride, void* state, const void* decay,
-                                      const void* cu_q, const void* positions, const void* slots, int n_seqs, int T,
-                                      int H, int D, int V, int num_decode, int dt, hipStream_t stream) {
-  if (n_seqs <= 0 || T <= 0) return 0;
-  if (D < 1 || D > 512 || V < 1) return -1;
+namespace {
+
+template <bool RET>
+int launch_linear(void* out, const void* qkv, long long stride, void* state, const void* decay, const void* cu_q,
+                  const void* positions, const void* slots, int n_seqs, int H, int D, int V, int dt, const HeadIn& in,
+                  hipStream_t stream) {
   if (D <= 256) {
     const dim3 wgrid(n_seqs * H, (V + kWideCols - 1) / kWideCols);
     const int nw = D > 64 ? 8 : 4;
     const int nr = (D + nw - 1) / nw;
 #define PKM_LIGHTW(NR, NW)                                                                                          \
-  PKM_DISPATCH(dt, E, lightning_wide_kernel<E, NR, NW><<<wgrid, 64 * NW, 0, stream>>>(                               \
+  PKM_DISPATCH(dt, E, lightning_wide_kernel<E, NR, NW, RET><<<wgrid, 64 * NW, 0, stream>>>(                          \
                           static_cast<float*>(out), static_cast<const E*>(qkv), stride, static_cast<float*>(state), \
                           static_cast<const float*>(decay), static_cast<const int*>(cu_q),                          \
-                          static_cast<const int*>(positions), static_cast<const int*>(slots), H, D, V))
+                          static_cast<const int*>(positions), static_cast<const int*>(slots), H, D, V, in))
     if (nw == 4) {
       if (nr <= 2) {
         PKM_LIGHTW(2, 4);
@@ -261,25 +289,36 @@ PK_EXPORT int pkm_lightning_attention(void* out, const void* qkv, long long stri
   const dim3 grid(n_seqs * H, (V + kCols - 1) / kCols);
   const int chunk = max(1, min(kMaxChunk, 15360 / (2 * D + kCols)));  // at most 60 KiB of LDS
   const size_t lds = static_cast<size_t>(chunk) * (2 * D + kCols) * sizeof(float);
-  const int nd = (D + 15) / 16;
-#define PKM_LIGHT(ND)                                                                                              \
-  PKM_DISPATCH(dt, E, lightning_kernel<E, ND><<<grid, 256, lds, stream>>>(                                          \
-                          static_cast<float*>(out), static_cast<const E*>(qkv), stride, static_cast<float*>(state), \
-                          static_cast<const float*>(decay), static_cast<const int*>(cu_q),                          \
-                          static_cast<const int*>(positions), static_cast<const int*>(slots), H, D, V, chunk))
-  if (nd <= 1) {
-    PKM_LIGHT(1);
-  } else if (nd <= 2) {
-    PKM_LIGHT(2);
-  } else if (nd <= 4) {
-    PKM_LIGHT(4);
-  } else if (nd <= 8) {
-    PKM_LIGHT(8);
-  } else if (nd <= 16) {
-    PKM_LIGHT(16);
-  } else {
-    PKM_LIGHT(32);
-  }
-#undef PKM_LIGHT
+  // heads of more than 256 key coordinates (narrower ones took the wider form)
+  PKM_DISPATCH(dt, E, lightning_kernel<E, 32, RET><<<grid, 256, lds, stream>>>(
+                          static_cast<float*>(out), static_cast<const E*>(qkv), stride, static_cast<float*>(state),
+                          static_cast<const float*>(decay), static_cast<const int*>(cu_q),
+                          static_cast<const int*>(positions), static_cast<const int*>(slots), H, D, V, chunk, in));
   return PK_CHECK_LAUNCH();
+}
+
+}  // namespace
+
+// out [T, H, V] fp32; qkv [T, H*D | H*D | H*V] projections (row stride `stride` elements);
+// state [slots, H, D, V] fp32; sequences 0..n_seqs-1 own tokens cu_q[s]..cu_q[s+1]-1.
+PK_EXPORT int pkm_lightning_attention(void* out, const void* qkv, long long stride, void* state, const void* decay,
+                                      const void* cu_q, const void* positions, const void* slots, int n_seqs, int T,
+                                      int H, int D, int V, int num_decode, int dt, hipStream_t stream) {
+  if (n_seqs <= 0 || T <= 0) return 0;
+  if (D < 1 || D > 512 || V < 1) return -1;
+  return launch_linear<false>(out, qkv, stride, state, decay, cu_q, positions, slots, n_seqs, H, D, V, dt,
+                              HeadIn{nullptr, 0, 0, nullptr, 1.f}, stream);
+}
+
+// the recurrence on plain projections: q and k turned by the position (table [rows, pairs, 2] fp32 or null), k
+// times k_scale
+PK_EXPORT int pkm_retention(void* out, const void* qkv, long long stride, void* state, const void* decay,
+                            const void* table, int pairs, int rows, float k_scale, const void* cu_q,
+                            const void* positions, const void* slots, int n_seqs, int T, int H, int D, int V, int dt,
+                            hipStream_t stream) {
+  if (n_seqs <= 0 || T <= 0) return 0;
+  if (D < 1 || D > 512 || V < 1 || 2 * pairs > D || (table && (rows < 1 || pairs < 1))) return -1;
+  return launch_linear<true>(out, qkv, stride, state, decay, cu_q, positions, slots, n_seqs, H, D, V, dt,
+                             HeadIn{static_cast<const float*>(table), pairs, rows, static_cast<const int*>(positions), k_scale},
+                             stream);
 }

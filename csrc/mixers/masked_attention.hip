@@ -11,7 +11,9 @@
 //   latent_query      [folded query | the head's rotated part turned by the position]
 //   masked_attention  query at position p sees keys lo(p) <= j <= p, lo(p) = max(0, p - window + 1,
 //                     floor(p / chunk) chunk); p_j = exp(s_j) / (exp(sink_h) + sum_j' exp(s_j')),
-//                     s = q . k * scale; o = sum_j p_j v_j.  Query head h reads key head h / (QH / KH)
+//                     s = q . k * scale; o = sum_j p_j v_j.  The first `keep` keys may stay visible behind
+//                     the band (j < keep, j <= p); a table may add bias[h][min(p - j, last)] to the scaled
+//                     score; o may be multiplied by one number (post).  Query head h reads key head h / (QH / KH)
 //                     and value head h / (QH / VH); the value may be the first V numbers of the key row.
 //   head_norm_gate    per (token, head): u / sqrt(mean(u^2) + eps) * w * post * act(gate), with u one
 //                     head's row or the difference first - coef * second of two attention maps
@@ -66,7 +68,7 @@ __global__ void __launch_bounds__(64)
 rotate_cache_kernel(T* __restrict__ q_out, const T* __restrict__ proj, int64_t stride, const int* __restrict__ positions,
                     const int* __restrict__ slot_mapping, const float* __restrict__ table, int pairs, int table_rows,
                     int halves, T* __restrict__ k_cache, T* __restrict__ v_cache, int QH, int KH, int VH, int D, int V,
-                    int bs, const float* __restrict__ q_norm, const float* __restrict__ k_norm, float eps) {
+                    int bs, const float* __restrict__ q_norm, const float* __restrict__ k_norm, int v_unit, float eps) {
   const int t = blockIdx.x, item = blockIdx.y, lane = threadIdx.x;
   const int slot = slot_mapping[t];
   const T* row = proj + static_cast<int64_t>(t) * stride;
@@ -85,7 +87,17 @@ rotate_cache_kernel(T* __restrict__ q_out, const T* __restrict__ proj, int64_t s
     const int g = item - QH - KH;
     const T* src = row + static_cast<int64_t>(QH + KH) * D + static_cast<int64_t>(g) * V;
     T* dst = v_cache + ((static_cast<int64_t>(slot / bs) * VH + g) * bs + slot % bs) * V;
-    for (int i = lane; i < V; i += 64) dst[i] = src[i];
+    if (v_unit) {
+      float ss = 0.f;
+      for (int i = lane; i < V; i += 64) {
+        const float x = ld<T>(src + i);
+        ss += x * x;
+      }
+      const float k = 1.f / sqrtf(pk::wave_sum(ss) / static_cast<float>(V) + eps);
+      for (int i = lane; i < V; i += 64) st<T>(dst + i, ld<T>(src + i) * k);
+    } else {
+      for (int i = lane; i < V; i += 64) dst[i] = src[i];
+    }
   }
 }
 
@@ -155,7 +167,10 @@ struct MaskedArgs {
   const float* sink;  // [QH] logits or null
   int n_seqs, QH, KH, VH, D, V, bs, BK;
   float scale;
-  int window, chunk;
+  int window, chunk, keep;
+  const float* bias;  // [QH, bias_n] added to the scaled scores by distance (the last entry for all beyond) or null
+  int bias_n;
+  float post;
   // decoded tokens on the matrix cores: the band's keys cut into n_parts runs of `part` keys,
   // partial sums in the workspace (merged by masked_merge_kernel)
   int part, n_parts;
@@ -168,6 +183,12 @@ __device__ __forceinline__ int first_key(int pos, int window, int chunk) {
   if (window > 0) lo = max(lo, pos - window + 1);
   if (chunk > 0) lo = max(lo, pos / chunk * chunk);
   return lo;
+}
+
+// The keys a tile of rows walks: kept tiles [0, kept) in front of the band's first tile, then the band.
+// Both bounds are multiples of the tile size, so tiles start at multiples of it whatever the rows are.
+__device__ __forceinline__ int kept_span(int keep, int k_begin, int bk) {
+  return keep > 0 ? min((keep + bk - 1) / bk * bk, k_begin) : 0;
 }
 
 // NV: output accumulators per thread = ceil(V / 16).  ALIAS: the value of a key is the first V
@@ -231,12 +252,15 @@ __global__ void __launch_bounds__(kThreads) masked_attention_kernel(MaskedArgs a
   const int last_pos = ctx - qlen + (min(row0 + kBQ, n_rows) - 1) / R;
   const int k_end = last_pos + 1;  // keys [k_begin, k_end) are visible to some row
   const int k_begin = first_pos >= 0 ? first_key(first_pos, a.window, a.chunk) / BK * BK : 0;
+  const int kept = kept_span(a.keep, k_begin, BK);
+  const float* my_bias = a.bias ? a.bias + static_cast<int64_t>(my_h) * a.bias_n : nullptr;
   float acc[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) acc[i] = 0.f;
   __syncthreads();
 
-  for (int k0 = k_begin; k0 < k_end; k0 += BK) {
+  for (int kv = 0; kv < kept + k_end - k_begin; kv += BK) {
+    const int k0 = kv < kept ? kv : k_begin + kv - kept;
     const int nk = min(BK, k_end - k0);
     for (int e = tid; e < BK * D; e += kThreads) {
       const int j = e / D, c = e - j * D;
@@ -267,7 +291,9 @@ __global__ void __launch_bounds__(kThreads) masked_attention_kernel(MaskedArgs a
       for (int c = 0; c < D; ++c) d += qr[c] * kr[c];
       d *= a.scale;
       const int key = k0 + j;
-      d = (j < nk && key <= my_pos && key >= my_lo) ? d : -INFINITY;
+      const bool seen = j < nk && key <= my_pos && (key >= my_lo || key < a.keep);
+      if (my_bias && seen) d += my_bias[min(my_pos - key, a.bias_n - 1)];
+      d = seen ? d : -INFINITY;
       ps[qi * BK + j] = d;
       tmax = fmaxf(tmax, d);
     }
@@ -302,7 +328,7 @@ __global__ void __launch_bounds__(kThreads) masked_attention_kernel(MaskedArgs a
     __syncthreads();
   }
   const float l = l_s[qi];
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float inv = l > 0.f ? a.post / l : 0.f;
   if (!live) return;
   const int64_t at = static_cast<int64_t>(q0 + my_tl) * a.out_ts + static_cast<int64_t>(my_h) * a.out_hs;
 #pragma unroll
@@ -374,9 +400,11 @@ constexpr float kLog2e = 1.4426950408889634f;
 
 __host__ __device__ __forceinline__ int quad_slot(int q) { return (q & 3) * 8 + 4 * (q >> 2); }  // slot of key 4 q
 
-// SPLIT: one token per sequence; blockIdx.z picks a run of a.part keys of the band and the
+// FINE: the softmax weights enter the value product as two bf16 parts (16 bits of them), and the kept keys
+// and the distance bias are built in.
+// SPLIT: one token per sequence; blockIdx.z picks a run of a.part of the walked keys and the
 // workgroup leaves (max, sum, unnormalised o) per row in the workspace (no sink: the merge adds it).
-template <int D, int V, int NW, bool ALIAS, bool SPLIT>
+template <int D, int V, int NW, bool ALIAS, bool SPLIT, bool FINE>
 __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedArgs a) {
   constexpr int NT = 64 * NW, BQ = 16 * NW, BK = 32, NKK = D / 32, NRT = V / 16, CS = D + 8, CT = BK + 8;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
@@ -410,12 +438,18 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
   const int my_pos = valid ? ctx - qlen + tl : -1;
   const int my_lo = valid ? first_key(my_pos, a.window, a.chunk) : 0x7fffffff;
   const int first_pos = ctx - qlen + row0 / R;
-  int max_pos = ctx - qlen + (min(row0 + BQ, n_rows) - 1) / R;
-  int k_begin = first_pos >= 0 ? first_key(first_pos, a.window, a.chunk) / BK * BK : 0;
+  const int max_pos = ctx - qlen + (min(row0 + BQ, n_rows) - 1) / R;
+  const int k_begin = first_pos >= 0 ? first_key(first_pos, a.window, a.chunk) / BK * BK : 0;
+  const int keep = FINE ? a.keep : 0;
+  const int kept = kept_span(keep, k_begin, BK);
+  // walked keys [w_begin, w_end): the kept tiles, then the band from its first tile
+  int w_begin = 0, w_end = kept + max_pos + 1 - k_begin;
   if (SPLIT) {
-    k_begin += blockIdx.z * a.part;
-    max_pos = min(max_pos, k_begin + a.part - 1);
+    w_begin = blockIdx.z * a.part;
+    w_end = min(w_end, w_begin + a.part);
   }
+  auto key_at = [&](int w) { return w < kept ? w : k_begin + w - kept; };
+  const float* my_bias = (FINE && a.bias) ? a.bias + static_cast<int64_t>(h) * a.bias_n : nullptr;
   const bf16_t* q = static_cast<const bf16_t*>(a.q);
   const bf16_t* kc = static_cast<const bf16_t*>(a.k_cache);
   const bf16_t* vc = static_cast<const bf16_t*>(a.v_cache);
@@ -462,8 +496,9 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
       }
     }
   };
-  if (k_begin <= max_pos) fetch(k_begin);
-  for (int k0 = k_begin; k0 <= max_pos; k0 += BK) {
+  if (w_begin < w_end) fetch(key_at(w_begin));
+  for (int w0 = w_begin; w0 < w_end; w0 += BK) {
+    const int k0 = key_at(w0);
 #pragma unroll
     for (int i = 0; i < KIT; ++i) {
       const int c = tid + NT * i;
@@ -491,8 +526,16 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
       }
     }
     __syncthreads();
-    if (k0 + BK <= max_pos) fetch(k0 + BK);
-    if (__any(my_pos >= k0 && my_lo <= k0 + BK - 1)) {
+    if (w0 + BK < w_end) fetch(key_at(w0 + BK));
+    if (__any(my_pos >= k0 && (my_lo <= k0 + BK - 1 || k0 < keep))) {
+      float bias[8];
+      if (FINE && my_bias) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int n_back = my_pos - (k0 + (e >> 2) * 16 + 4 * g + (e & 3));
+          bias[e] = my_bias[min(max(n_back, 0), a.bias_n - 1)] * kLog2e;
+        }
+      }
       pk::f32x4 sa[2] = {pk::f32x4{0.f, 0.f, 0.f, 0.f}, pk::f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
       for (int sub = 0; sub < 2; ++sub) {
@@ -506,7 +549,9 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const int key = k0 + (e >> 2) * 16 + 4 * g + (e & 3);
-        sc[e] = (key <= my_pos && key >= my_lo) ? sa[e >> 2][e & 3] * sl2 : -INFINITY;
+        float v = sa[e >> 2][e & 3] * sl2;
+        if (FINE && my_bias) v += bias[e];
+        sc[e] = (key <= my_pos && (key >= my_lo || key < keep)) ? v : -INFINITY;
         tmax = fmaxf(tmax, sc[e]);
       }
       tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
@@ -535,6 +580,16 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
 #pragma unroll
       for (int rt = 0; rt < NRT; ++rt)
         o[rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pk::ld8(vr + rt * 16 * CT), pb, o[rt], 0, 0, 0);
+      if (FINE) {  // what rounding the weights to bf16 left over
+        pk::u32x4 lw;
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          lw[e] = pk::pack2(p[2 * e] - __uint_as_float(pw[e] << 16), p[2 * e + 1] - __uint_as_float(pw[e] & 0xffff0000u));
+        const pk::bf16x8_t lb = __builtin_bit_cast(pk::bf16x8_t, lw);
+#pragma unroll
+        for (int rt = 0; rt < NRT; ++rt)
+          o[rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pk::ld8(vr + rt * 16 * CT), lb, o[rt], 0, 0, 0);
+      }
     }
     __syncthreads();
   }
@@ -552,7 +607,7 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
     return;
   }
   if (valid) {
-    const float inv = l_run > 0.f ? 1.f / l_run : 0.f;
+    const float inv = l_run > 0.f ? a.post / l_run : 0.f;
     const int64_t at = static_cast<int64_t>(q0 + tl) * a.out_ts + static_cast<int64_t>(h) * a.out_hs + 4 * g;
 #pragma unroll
     for (int rt = 0; rt < NRT; ++rt) {
@@ -575,7 +630,7 @@ template <typename T>
 __global__ void __launch_bounds__(128)
 masked_merge_kernel(void* __restrict__ out, int64_t out_ts, int64_t out_hs, int out_f32, const float* __restrict__ ws_o,
                     const float* __restrict__ ws_ml, const int* __restrict__ cu_q, const float* __restrict__ sink,
-                    int n_parts, int QH, int V) {
+                    int n_parts, int QH, int V, float post) {
   __shared__ float wgt[64];
   const int s = blockIdx.x, h = blockIdx.y;
   const int tok = cu_q[s];
@@ -589,7 +644,7 @@ masked_merge_kernel(void* __restrict__ out, int64_t out_ts, int64_t out_hs, int 
     const float w = m == -INFINITY ? 0.f : exp2f(m - M);
     float L = pk::wave_sum(w * l);
     if (sink) L += exp2f(sk - M);
-    wgt[p] = L > 0.f ? w / L : 0.f;
+    wgt[p] = L > 0.f ? w * post / L : 0.f;
   }
   __syncthreads();
   const int64_t at = static_cast<int64_t>(tok) * out_ts + static_cast<int64_t>(h) * out_hs;
@@ -605,10 +660,10 @@ masked_merge_kernel(void* __restrict__ out, int64_t out_ts, int64_t out_hs, int 
   }
 }
 
-template <int D, int V, int NW, bool ALIAS, bool SPLIT>
+template <int D, int V, int NW, bool ALIAS, bool SPLIT, bool FINE>
 int launch_mfma_one(const MaskedArgs& a, int T, hipStream_t stream) {
   constexpr size_t lds = (32 * (D + 8) + V * 40) * sizeof(bf16_t);
-  auto kern = masked_attention_mfma_kernel<D, V, NW, ALIAS, SPLIT>;
+  auto kern = masked_attention_mfma_kernel<D, V, NW, ALIAS, SPLIT, FINE>;
   if (lds > 60 * 1024) {
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize,
                                              static_cast<int>(lds));
@@ -629,10 +684,10 @@ bool mfma_sizes(int D, int V, bool alias) {
 }
 
 // returns -100 when the sizes are not among those the matrix-core kernel is built for
-template <bool SPLIT>
+template <bool SPLIT, bool FINE>
 int launch_mfma(const MaskedArgs& a, int T, bool alias, hipStream_t stream) {
 #define PKM_MM(DD, VV, NW, NWS, AL) \
-  if (a.D == DD && a.V == VV && alias == AL) return launch_mfma_one<DD, VV, (SPLIT ? NWS : NW), AL, SPLIT>(a, T, stream);
+  if (a.D == DD && a.V == VV && alias == AL) return launch_mfma_one<DD, VV, (SPLIT ? NWS : NW), AL, SPLIT, FINE>(a, T, stream);
   // waves per workgroup for prompt portions / for decoded tokens (one 16-row tile computes there:
   // fewer, less loaded waves stage the tiles faster for the wide rows)
   PKM_MM(64, 64, 8, 8, false)
@@ -692,11 +747,11 @@ head_norm_gate_kernel(OT* __restrict__ out, int64_t out_stride, const float* __r
 }  // namespace
 
 // proj [T, QH*D | KH*D | VH*V] rows `stride` elements apart; table [table_rows, pairs, 2] fp32 or null;
-// q_norm / k_norm [D] fp32 or null: unit RMS times the weight before the rotation
+// q_norm / k_norm [D] fp32 or null: unit RMS times the weight before the rotation; v_unit: v set to unit RMS
 PK_EXPORT int pkm_rotate_cache(void* q_out, const void* proj, long long stride, const void* positions,
                                const void* slot_mapping, const void* table, int pairs, int table_rows, int halves,
                                void* k_cache, void* v_cache, int T, int QH, int KH, int VH, int D, int V, int bs,
-                               const void* q_norm, const void* k_norm, float eps, int dt, hipStream_t stream) {
+                               const void* q_norm, const void* k_norm, int v_unit, float eps, int dt, hipStream_t stream) {
   if (T <= 0) return 0;
   if (D < 1 || V < 1 || 2 * pairs > D || (table && table_rows < 1) || bs < 1) return -1;
   const dim3 grid(T, QH + KH + VH);
@@ -704,18 +759,18 @@ PK_EXPORT int pkm_rotate_cache(void* q_out, const void* proj, long long stride, 
                           static_cast<E*>(q_out), static_cast<const E*>(proj), stride, static_cast<const int*>(positions),
                           static_cast<const int*>(slot_mapping), static_cast<const float*>(table), pairs, table_rows,
                           halves, static_cast<E*>(k_cache), static_cast<E*>(v_cache), QH, KH, VH, D, V, bs,
-                          static_cast<const float*>(q_norm), static_cast<const float*>(k_norm), eps));
+                          static_cast<const float*>(q_norm), static_cast<const float*>(k_norm), v_unit, eps));
   return PK_CHECK_LAUNCH();
 }
 
-// proj [T, Q | R | Dr]; cq [T, Q] (null with Q = 0); cache rows [slots, R + Dr]
+// proj [T, Q | R | Dr]; cq [T, Q] (null with Q = 0); cache rows [slots, R + Dr] (null: only the query latent)
 PK_EXPORT int pkm_latent_in(void* cq, void* cache, const void* proj, long long stride, int Q, int R, int Dr, const void* wq,
                             const void* wkv, float eps, const void* positions, const void* slot_mapping,
                             const void* table, int pairs, int table_rows, int halves, int T, int bs, int dt,
                             hipStream_t stream) {
   if (T <= 0) return 0;
   if (R < 1 || Q < 0 || Dr < 0 || 2 * pairs > Dr || (table && table_rows < 1) || (Q > 0 && (!cq || !wq))) return -1;
-  const dim3 grid(T, 2);
+  const dim3 grid(T, cache ? 2 : 1);  // no cache: the query latent alone (the row holds nothing else)
   PKM_DISPATCH(dt, E, latent_in_kernel<E><<<grid, 256, 0, stream>>>(
                           static_cast<E*>(cq), static_cast<E*>(cache), static_cast<const E*>(proj), stride, Q, R, Dr,
                           static_cast<const float*>(wq), static_cast<const float*>(wkv), eps,
@@ -738,16 +793,19 @@ PK_EXPORT int pkm_latent_query(void* out, const void* q_lat, const void* q, cons
   return PK_CHECK_LAUNCH();
 }
 
-// v_cache == k_cache: the value of a key is the first V numbers of its key row
+// v_cache == k_cache: the value of a key is the first V numbers of its key row.  keep: keys below it stay visible;
+// bias [QH, bias_n] fp32 or null; post multiplies the result; fine: softmax weights to 16 bits on the matrix cores
+// (always with keep or bias)
 PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs, int out_dt, const void* q, int q_dt,
                                    const void* k_cache, const void* v_cache, int v_width, const void* block_tables,
                                    long long bt_stride, const void* cu_q, const void* context_lens, const void* sink,
                                    int n_seqs, int T, int QH, int KH, int VH, int D, int V, int bs, float scale, int window,
-                                   int chunk, int num_decode, void* ws_o, void* ws_ml, int part, int n_parts, int dt,
-                                   hipStream_t stream) {
+                                   int chunk, int keep, const void* bias, int bias_n, float post, int fine, int num_decode,
+                                   void* ws_o, void* ws_ml, int part, int n_parts, int dt, hipStream_t stream) {
   if (n_seqs <= 0 || T <= 0) return 0;
   if (KH < 1 || VH < 1 || QH % KH || KH % VH || V < 1 || V > 512 || V > v_width || D < 1) return -1;
   if ((q_dt != dt && q_dt != kF32) || (out_dt != dt && out_dt != kF32)) return -1;
+  if (keep < 0 || (bias && bias_n < 1)) return -1;
   const bool alias = v_cache == k_cache;
   if (alias && (KH != VH || v_width != D)) return -1;
   const int bk = key_tile(D, V, alias);
@@ -755,9 +813,11 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
   MaskedArgs a{out, out_ts, out_hs, out_dt == kF32, q, q_dt == kF32, k_cache, v_cache, v_width,
                static_cast<const int*>(block_tables), bt_stride, static_cast<const int*>(cu_q),
                static_cast<const int*>(context_lens), static_cast<const float*>(sink), n_seqs, QH, KH, VH, D, V, bs, bk,
-               scale, window, chunk, 0, 1, nullptr, nullptr};
+               scale, window, chunk, keep, static_cast<const float*>(bias), bias_n, post, 0, 1, nullptr, nullptr};
+  const bool finer = fine || keep > 0 || bias;
   const int R = QH / KH;
-  if (g_masked_mfma && dt == kBF16 && q_dt == kBF16 && bs % 32 == 0 && v_width % 8 == 0 && mfma_sizes(D, V, alias)) {
+  if (g_masked_mfma && dt == kBF16 && q_dt == kBF16 && bs % 32 == 0 && v_width % 8 == 0 && out_ts % 4 == 0 && out_hs % 4 == 0 &&
+      mfma_sizes(D, V, alias)) {
     // the first num_decode sequences hold one token each: their bands are cut into runs when a
     // workspace is given (ws_o [num_decode, n_parts, QH, V], ws_ml [num_decode, n_parts, QH, 2] fp32)
     const int nd = (ws_o && ws_ml && n_parts > 1) ? (num_decode < n_seqs ? num_decode : n_seqs) : 0;
@@ -769,10 +829,10 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
       d.n_parts = n_parts;
       d.ws_o = static_cast<float*>(ws_o);
       d.ws_ml = static_cast<float*>(ws_ml);
-      int rc = launch_mfma<true>(d, nd, alias, stream);
+      int rc = finer ? launch_mfma<true, true>(d, nd, alias, stream) : launch_mfma<true, false>(d, nd, alias, stream);
       if (rc) return rc;
       masked_merge_kernel<bf16_t><<<dim3(nd, QH), 128, 0, stream>>>(out, out_ts, out_hs, a.out_f32, d.ws_o, d.ws_ml, d.cu_q,
-                                                                    d.sink, n_parts, QH, V);
+                                                                    d.sink, n_parts, QH, V, post);
       rc = PK_CHECK_LAUNCH();
       if (rc) return rc;
     }
@@ -782,7 +842,7 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
       p.block_tables += static_cast<int64_t>(nd) * bt_stride;
       p.cu_q += nd;
       p.context_lens += nd;
-      return launch_mfma<false>(p, T - nd, alias, stream);
+      return finer ? launch_mfma<false, true>(p, T - nd, alias, stream) : launch_mfma<false, false>(p, T - nd, alias, stream);
     }
     return 0;
   }
@@ -798,14 +858,15 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
 
 // Keys per run of a decoded token's band (a multiple of 32), 0: no split.  `capacity`: the most
 // cached tokens of a sequence; the band spans at most window + 31 / chunk + 31 keys from its
-// aligned start.  Runs are at least 64 keys, at most 64 of them, and aim at ~512 workgroups per launch.
+// aligned start, with the kept keys' tiles in front.  Runs are at least 64 keys, at most 64 of them, and aim at ~512 workgroups per launch.
 PK_EXPORT int pkm_masked_decode_part(int nd, int QH, int KH, int D, int V, int alias, int bs, int capacity, int window,
-                                     int chunk, int dt) {
+                                     int chunk, int keep, int dt) {
   if (!g_masked_mfma || dt != kBF16 || bs % 32 || nd <= 0 || !mfma_sizes(D, V, alias != 0)) return 0;
   int span = capacity;
   if (window > 0 && window + 31 < span) span = window + 31;
   if (chunk > 0 && chunk + 31 < span) span = chunk + 31;
-  span = (span + 31) / 32 * 32;
+  span = (span + 31) / 32 * 32 + (keep + 31) / 32 * 32;
+  if (span > (capacity + 31) / 32 * 32) span = (capacity + 31) / 32 * 32;
   const int wgs = nd * KH;
   int want = (512 + wgs - 1) / wgs;  // runs wanted
   if (want > 64) want = 64;

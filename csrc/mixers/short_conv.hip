@@ -76,17 +76,65 @@ conv_state_kernel(float* __restrict__ state, const TI* __restrict__ x, int64_t x
   }
 }
 
+// Steps in which every sequence holds one token: one thread per (sequence, channel) filters and moves
+// the slot's rows (row j is read before row j - 1 takes it).  The same sums in the same order.
+template <typename TI, typename TO>
+__global__ void __launch_bounds__(256)
+conv_step_kernel(TO* __restrict__ out, const TI* __restrict__ x, int64_t xs, const float* __restrict__ in_bias,
+                 const float* __restrict__ taps, int K, const float* __restrict__ bias, float* __restrict__ state,
+                 const int* __restrict__ positions, const int* __restrict__ slots, int C, int act, int residual) {
+  const int t = blockIdx.x;
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= C) return;
+  const int slot = slots[t];
+  const bool carry = slot >= 0 && positions[t] > 0;
+  float* rows = slot >= 0 ? state + static_cast<int64_t>(slot) * (K - 1) * C + c : nullptr;
+  const float* w = taps + static_cast<int64_t>(c) * K;
+  const float xv = ld<TI>(x + static_cast<int64_t>(t) * xs + c) + (in_bias ? in_bias[c] : 0.f);
+  float acc = 0.f;
+  for (int j = 0; j < K - 1; ++j) {
+    const float v = carry ? rows[static_cast<int64_t>(j) * C] : 0.f;
+    acc += w[j] * v;
+    if (rows && j > 0) rows[static_cast<int64_t>(j - 1) * C] = v;
+  }
+  if (rows) rows[static_cast<int64_t>(K - 2) * C] = xv;
+  acc += w[K - 1] * xv;
+  if (bias) acc += bias[c];
+  if (act == kActSilu) acc = acc * sigmoidf(acc);
+  if (residual) acc += xv;
+  st<TO>(out + static_cast<int64_t>(t) * C + c, acc);
+}
+
 }  // namespace
 
+// single: every sequence holds one token (n_seqs == T).
 // x [T, C] rows x_stride elements apart (x_dt); out [T, C] contiguous (out_dt); taps [C, K] fp32; in_bias, bias [C]
 // fp32 or null; state [slots, K - 1, C] fp32 (null with K = 1), brought up to date after the outputs
 PK_EXPORT int pkm_causal_conv(void* out, int out_dt, const void* x, int x_dt, long long x_stride, const void* in_bias,
                               const void* taps, int K, const void* bias, void* state, const void* cu_q,
                               const void* positions, const void* slots, const void* token_seq, int n_seqs, int T, int C,
-                              int act, int residual, hipStream_t stream) {
+                              int act, int residual, int single, hipStream_t stream) {
   if (T <= 0) return 0;
   if (K < 1 || C < 1 || (K > 1 && state == nullptr) || x_stride < C) return -1;
+  if (single && n_seqs != T) return -1;
   const dim3 grid(T, (C + 255) / 256);
+  if (single && K > 1) {
+#define PKM_CS(TI)                                                                                                     \
+  PKM_DISPATCH(out_dt, O, conv_step_kernel<TI, O><<<grid, 256, 0, stream>>>(                                             \
+                              static_cast<O*>(out), static_cast<const TI*>(x), x_stride, static_cast<const float*>(in_bias), \
+                              static_cast<const float*>(taps), K, static_cast<const float*>(bias),                         \
+                              static_cast<float*>(state), static_cast<const int*>(positions),                              \
+                              static_cast<const int*>(slots), C, act, residual))
+    if (x_dt == kF32) {
+      PKM_CS(float);
+    } else if (x_dt == kBF16) {
+      PKM_CS(bf16_t);
+    } else {
+      return -2;
+    }
+#undef PKM_CS
+    return PK_CHECK_LAUNCH();
+  }
 #define PKM_CC(TI)                                                                                                       \
   PKM_DISPATCH(out_dt, O, causal_conv_kernel<TI, O><<<grid, 256, 0, stream>>>(                                             \
                               static_cast<O*>(out), static_cast<const TI*>(x), x_stride, static_cast<const float*>(in_bias), \

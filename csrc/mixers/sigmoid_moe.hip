@@ -97,12 +97,12 @@ __device__ __forceinline__ bool find_tile(const int* offsets, int E, int tile, i
 // C[r, n] = sum_k A[arow(r), k] * B[e][n, k]   (B: [E, N, K]); DUAL: a second B and a gated
 // epilogue: with slot_scale the scaled SiLU product, without it the clamped product
 // min(g, limit) * sigmoid(1.702 min(g, limit)) * (clamp(u, -limit, limit) + 1), or with limit <= 0 the plain
-// SiLU product silu(g) * u.  256 threads: thread (ty, tx) owns rows ty, ty + 16 and columns tx, tx + 16.
+// SiLU product silu(g) * u.  A single B with relu2: max(v, 0)^2.  256 threads: thread (ty, tx) owns rows ty, ty + 16 and columns tx, tx + 16.
 template <typename T, typename TA, typename TC, bool DUAL>
 __global__ void __launch_bounds__(256)
 grouped_rows_kernel(TC* __restrict__ C, const TA* __restrict__ A, const T* __restrict__ B0, const T* __restrict__ B1,
                     const int* __restrict__ offsets, const int* __restrict__ sorted_slots,
-                    const float* __restrict__ slot_scale, int top, int E, int N, int K, float limit) {
+                    const float* __restrict__ slot_scale, int top, int E, int N, int K, float limit, int relu2 = 0) {
   __shared__ float as[kBM][kBK + 1];
   __shared__ float b0s[kBN][kBK + 1];
   __shared__ float b1s[DUAL ? kBN : 1][kBK + 1];
@@ -166,6 +166,9 @@ grouped_rows_kernel(TC* __restrict__ C, const TA* __restrict__ A, const T* __res
         v = g * sigmoidf(1.702f * g) * (u + 1.f);
       } else if (DUAL) {
         v = v * sigmoidf(v) * acc1[i][j];
+      } else if (relu2) {
+        v = fmaxf(v, 0.f);
+        v *= v;
       }
       st<TC>(C + static_cast<int64_t>(r) * N + n, v);
     }
@@ -271,6 +274,18 @@ PK_EXPORT int pkm_expert_gate_up_clamped(void* h, const void* x, const void* gat
                           static_cast<T*>(h), static_cast<const T*>(x), static_cast<const T*>(gate),
                           static_cast<const T*>(up), static_cast<const int*>(offsets),
                           static_cast<const int*>(sorted_slots), nullptr, top, E, F, W, limit));
+  return PK_CHECK_LAUNCH();
+}
+
+// ungated experts: h [n_rows, F] = max(up x, 0)^2
+PK_EXPORT int pkm_expert_up_relu2(void* h, const void* x, const void* up, const void* offsets, const void* sorted_slots,
+                                  int n_rows, int top, int E, int F, int W, int dt, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  const dim3 grid((n_rows + kBM - 1) / kBM + E, (F + kBN - 1) / kBN);
+  PKM_DISPATCH(dt, T, grouped_rows_kernel<T, T, T, false><<<grid, 256, 0, stream>>>(
+                          static_cast<T*>(h), static_cast<const T*>(x), static_cast<const T*>(up), nullptr,
+                          static_cast<const int*>(offsets), static_cast<const int*>(sorted_slots), nullptr, top, E, F, W,
+                          0.f, 1));
   return PK_CHECK_LAUNCH();
 }
 

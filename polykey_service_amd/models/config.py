@@ -92,7 +92,9 @@ class LatentAttentionSpec:
     Optional parts (0 / None: absent): queries through a normed latent of ``q_rank`` numbers; one
     rotated key part of ``rot_dim`` numbers per token shared by all heads (cached beside the
     latent) against ``rot_dim`` rotated query numbers per head; a sliding window of ``window``
-    positions; one learned sink logit per head in the softmax denominator."""
+    positions; one learned sink logit per head in the softmax denominator.  ``kv_from`` >= 0: the layer
+    has no latent of its own and reads the cache of that layer; ``fine``: softmax weights kept to 16
+    bits on the matrix cores."""
     heads: int
     dim: int        # unrotated query / key size per head
     vdim: int       # value size per head
@@ -103,6 +105,8 @@ class LatentAttentionSpec:
     rot: Optional["RotarySpec"] = None
     window: int = 0
     sink: bool = False
+    kv_from: int = -1
+    fine: bool = False
 
 
 @dataclasses.dataclass(frozen=True)
@@ -741,9 +745,221 @@ class BibezenConfig:
                    residual_mult=0.5, embed_scale=float(width) ** 0.5, canon_taps=3)
 
 
+@dataclasses.dataclass(frozen=True)
+class BiasedAttentionSpec:
+    """Grouped-query softmax attention without rotation: weighted unit-RMS query / key heads, plain
+    unit-RMS value heads, a learned bias by distance bucket (logarithmic up to ``bias_max``), the last
+    ``window`` keys visible (0: all) and the first ``keep`` ones always."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    bias_max: int
+    window: int = 0
+    keep: int = 0
+
+
+@dataclasses.dataclass(frozen=True)
+class GatedRecurrenceSpec:
+    """Real-gated linear recurrence of ``width`` channels behind a causal filter of ``conv`` taps, its
+    gates block-diagonal in ``blocks`` parts, beside a GELU branch."""
+    width: int
+    blocks: int
+    conv: int
+
+
+@dataclasses.dataclass(frozen=True)
+class RetentionSpec:
+    """Linear attention with one constant decay per head on plain projections, rotated queries and
+    keys (keys times dim^-1/2), unit RMS per head and a SiLU gate."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+    rot: Optional[RotarySpec] = None
+
+
+@dataclasses.dataclass(frozen=True)
+class XieluFFSpec:
+    """down(xIELU(up x)) with two learned numbers per layer."""
+    ff: int
+
+
+@dataclasses.dataclass(frozen=True)
+class GroupedMoESpec:
+    """Ungated squared-ReLU experts chosen by softmax score plus a learned correction inside the
+    ``keep`` best of ``groups`` expert groups, weighted by the score alone."""
+    experts: int
+    top: int
+    ff: int
+    groups: int = 1
+    keep: int = 1
+
+
+@dataclasses.dataclass(frozen=True)
+class LefuvikConfig:
+    """Lefuvik: a normed embedding starts one fp32 residual stream; pre-norm sublayers (norm weights
+    stored around zero) whose outputs are scaled coordinate by coordinate; a per-layer token input
+    (``side_dim`` numbers per token and layer; 0: none) behind the feed-forward; mixers are ``parallel``
+    (distance-biased attention beside a gated linear recurrence), ``retention`` or ``latent_attention``
+    (optionally on an earlier layer's cache); feed-forwards are dense xIELU, a group-routed mixture of
+    squared-ReLU experts, or none.  Logits reuse the embedding table, capped by tanh.  Read from a
+    checkpoint folder's config.json ("architecture": "Lefuvik")."""
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: tuple
+    rms_eps: float
+    side_dim: int = 0
+    logit_softcap: float = 0.0
+    buckets: int = 32               # distance buckets of random weights (a checkpoint's table has its own)
+    max_position: int = 1 << 20
+    bos_token_id: int = 0
+    eos_token_id: int = -1
+    init_std: float = 0.05
+    family: str = "lefuvik"
+    is_moe: bool = False
+    experts_per_token: int = 0
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def runs(self) -> tuple:
+        return tuple(range(len(self.layers)))
+
+    @property
+    def needs_state(self) -> bool:
+        return any(l.type != "latent_attention" for l in self.layers)
+
+    def num_params(self) -> int:
+        W, D = self.hidden_size, self.side_dim
+        n = self.vocab_size * (W + D * len(self.layers)) + 2 * W
+        for l in self.layers:
+            m, f = l.mixer, l.mlp
+            n += W * (4 if f is not None else 2) + ((2 * D + 1) * W if D else 0)
+            if l.type == "parallel":
+                a, b = m.left, m.right
+                n += W * (a.heads * (a.dim + a.vdim) + a.kv_heads * (a.dim + a.vdim)) + 2 * a.dim + self.buckets * a.heads
+                n += 3 * W * b.width + b.width * (b.conv + 6 + 2 * (b.width // b.blocks))
+            elif l.type == "retention":
+                n += W * m.heads * (2 * m.dim + 3 * m.vdim)
+            else:
+                n += W * m.q_rank + m.q_rank * (1 + m.heads * (m.dim + m.rot_dim)) + W * m.heads * m.vdim
+                n += m.kv_rank * m.heads * (m.dim + m.vdim)
+                n += W * (m.kv_rank + m.rot_dim) + m.kv_rank if m.kv_from < 0 else 0
+            if isinstance(f, XieluFFSpec):
+                n += 2 * W * f.ff + 2
+            elif f is not None:
+                n += f.experts * (2 * f.ff * W + W + 1)
+        return n
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        n = 0
+        for l in self.layers:
+            if l.type == "parallel":
+                n += l.mixer.left.kv_heads * (l.mixer.left.dim + l.mixer.left.vdim)
+            elif l.type == "latent_attention" and l.mixer.kv_from < 0:
+                n += l.mixer.kv_rank + l.mixer.rot_dim
+        return n * dtype_bytes
+
+    @staticmethod
+    def _rot(r: Optional[dict], width: int, halves: bool) -> Optional[RotarySpec]:
+        if not r:
+            return None
+        rot = RotarySpec(int(r["dims"]), float(r["base"]), None, halves=halves)
+        if rot.dims % 2 or rot.dims > width:
+            raise ValueError("Lefuvik: rot.dims must be even and fit the rotated vector")
+        return rot if rot.dims else None
+
+    @classmethod
+    def _mixer(cls, kind: str, m: dict, before: list):
+        if kind == "parallel":
+            a, b = m["left"], m["right"]
+            mask = a.get("mask") or {}
+            left = BiasedAttentionSpec(int(a["heads"]), int(a.get("kv_heads", a["heads"])), int(a["dim"]),
+                                       int(a.get("vdim", a["dim"])), float(a["scale"]), int(a["bias_max"]),
+                                       int(mask.get("size") or 0), int(mask.get("keep_first") or 0))
+            right = GatedRecurrenceSpec(int(b["width"]), int(b["blocks"]), int(b["conv"]))
+            if left.heads % left.kv_heads or right.width % right.blocks or right.conv < 1:
+                raise ValueError("Lefuvik: heads must divide by kv_heads, width by blocks, conv be at least 1")
+            return ParallelSpec(left, right, float(m.get("left_scale", 1.0)), float(m.get("right_scale", 1.0)))
+        if kind == "retention":
+            s = RetentionSpec(int(m["heads"]), int(m["dim"]), int(m.get("vdim", m["dim"])), tuple(float(d) for d in m["decay"]),
+                              cls._rot(m.get("rot"), int(m["dim"]), True))
+            if len(s.decay) != s.heads:
+                raise ValueError("Lefuvik: a retention mixer needs one decay per head")
+            return s
+        if kind == "latent_attention":
+            src = m.get("kv_from")
+            src = -1 if src is None else int(src)
+            s = LatentAttentionSpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), int(m["kv_rank"]), float(m["scale"]),
+                                    int(m["q_rank"]), int(m["rot_dim"]), cls._rot(m.get("rot"), int(m["rot_dim"]), False),
+                                    int((m.get("mask") or {}).get("size") or 0), False, src, True)
+            if src >= 0:
+                o = before[src].mixer if src < len(before) else None
+                if not isinstance(o, LatentAttentionSpec) or o.kv_from >= 0 or (o.kv_rank, o.rot_dim) != (s.kv_rank, s.rot_dim):
+                    raise ValueError("Lefuvik: kv_from must name an earlier latent layer of its own with the same sizes")
+            return s
+        raise ValueError(f"Lefuvik: unknown mixer type {kind!r}")
+
+    @staticmethod
+    def _mlp(f: Optional[dict]):
+        if f is None:
+            return None
+        if f.get("kind") == "dense":
+            return XieluFFSpec(int(f["ff"]))
+        if f.get("kind") != "moe":
+            raise ValueError(f"Lefuvik: unknown feed-forward kind {f.get('kind')!r}")
+        r = f["router"]
+        g = r.get("groups") or {}
+        s = GroupedMoESpec(int(r["experts"]), int(r["top"]), int(f["expert"]["ff"]), int(g.get("count", 1)), int(g.get("keep", 1)))
+        if s.experts % s.groups or not 1 <= s.keep <= s.groups or not 1 <= s.top <= s.keep * (s.experts // s.groups):
+            raise ValueError("Lefuvik: the expert groups must be equal and hold enough experts for `top`")
+        return s
+
+    @classmethod
+    def from_json(cls, c: dict, name: str = "lefuvik") -> "LefuvikConfig":
+        layers = []
+        for l in c["layers"]:
+            layers.append(LayerSpec(l["type"], cls._mixer(l["type"], l["mixer"], layers), cls._mlp(l.get("mlp"))))
+        return cls(name=name, vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), layers=tuple(layers),
+                   rms_eps=float(c["norm"]["eps"]), side_dim=int((c.get("token_side") or {}).get("dim") or 0),
+                   logit_softcap=float(c.get("logit_softcap") or 0.0))
+
+    @classmethod
+    def uniform(cls, name: str, vocab: int, width: int, pattern: str, heads: int, kv_heads: int, dim: int, ff: int,
+                experts: int = 16, top: int = 2, expert_ff: int = 2304, groups: int = 4, keep: int = 2, side_dim: int = 256,
+                kv_rank: int = 512, q_rank: int = 1024, rot_dim: int = 64, window: int = 1024, first: int = 64,
+                bias_max: int = 1024, rec_blocks: int = 16) -> "LefuvikConfig":
+        """``pattern``: one letter per layer, P parallel / R retention / M latent attention / S latent
+        attention on the last M layer's cache; upper case with the mixture, lower case with the dense
+        feed-forward."""
+        layers, last = [], -1
+        for i, ch in enumerate(pattern):
+            up = ch.upper()
+            if up == "P":
+                mixer = ParallelSpec(BiasedAttentionSpec(heads, kv_heads, dim, dim, dim ** -0.5, bias_max, window, first),
+                                     GatedRecurrenceSpec(width, rec_blocks, 4), 0.7, 0.7)
+            elif up == "R":
+                mixer = RetentionSpec(heads, dim, dim, tuple(1.0 - 2.0 ** (-5 - 6 * h / max(heads - 1, 1)) for h in range(heads)),
+                                      RotarySpec(dim, 1e4, None, True))
+            else:
+                mixer = LatentAttentionSpec(heads, dim, dim, kv_rank, (dim + rot_dim) ** -0.5, q_rank, rot_dim,
+                                            RotarySpec(rot_dim, 1e4, None, False), window, False, last if up == "S" else -1, True)
+                last = i if up == "M" else last
+            mlp = GroupedMoESpec(experts, top, expert_ff, groups, keep) if ch.isupper() else XieluFFSpec(ff)
+            layers.append(LayerSpec({"P": "parallel", "R": "retention"}.get(up, "latent_attention"), mixer, mlp))
+        return cls(name=name, vocab_size=vocab, hidden_size=width, layers=tuple(layers), rms_eps=1e-5, side_dim=side_dim,
+                   logit_softcap=30.0)
+
+
 # config.json "architecture" -> reader (checkpoints that are not HF Llama / Mixtral folders)
 ARCHITECTURES = {"Sapapel": SapapelConfig.from_json, "Kivezen": KivezenConfig.from_json,
-                 "Nopunex": NopunexConfig.from_json, "Bibezen": BibezenConfig.from_json}
+                 "Nopunex": NopunexConfig.from_json, "Bibezen": BibezenConfig.from_json,
+                 "Lefuvik": LefuvikConfig.from_json}
 
 PRESETS["tiny-sapapel"] = SapapelConfig.uniform("tiny-sapapel", 512, 128, 3, 4, 16, 32, 48, 64, 6, 2)
 # speed measurements (random weights): layer shapes of small production MoE models, and the
@@ -778,6 +994,17 @@ PRESETS["tiny-bibezen"] = BibezenConfig.uniform("tiny-bibezen", 512, 128, "wPSp"
 # the same width, depth, heads, KV heads, head size, experts and expert size
 PRESETS["bibezen-2k"] = BibezenConfig.uniform("bibezen-2k", 32000, 2048, "WPPPSPPP", 16, 4, 128, 4096, 16, 2, 1536)
 PRESETS["bibezen-4k"] = BibezenConfig.uniform("bibezen-4k", 32000, 4096, "WPSP", 32, 8, 128, 8192, 8, 2, 2048)
+
+
+PRESETS["tiny-lefuvik"] = LefuvikConfig.uniform("tiny-lefuvik", 512, 128, "pRMSP", 4, 2, 32, 256, 6, 2, 64, 3, 2, side_dim=8,
+                                                kv_rank=48, q_rank=64, rot_dim=8, window=40, first=10, bias_max=50,
+                                                rec_blocks=4)
+# speed measurements beside bibezen-2k / bibezen-4k (the closest family: an attention and a recurrent
+# branch side by side in parallel layers, a recurrent mixer of its own, a mixture feed-forward) and
+# nopunex-2k / -4k (windowed latent attention): the same width, depth, heads, KV heads and head size;
+# ungated experts half as wide again as the gated ones (equal weights per expert)
+PRESETS["lefuvik-2k"] = LefuvikConfig.uniform("lefuvik-2k", 32000, 2048, "RPMPRPSP", 16, 4, 128, 6144)
+PRESETS["lefuvik-4k"] = LefuvikConfig.uniform("lefuvik-4k", 32000, 4096, "RPMP", 32, 8, 128, 12288, 8, 2, 3072, rec_blocks=32)
 
 
 def get_config(name_or_path: str):

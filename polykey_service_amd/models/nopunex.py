@@ -101,7 +101,8 @@ class DiffAttention(nn.Module):
 
 class WindowLatentAttention(nn.Module):
     """Weights of one latent-attention mixer with a query latent, a shared rotated key part, a
-    sliding window and sink logits.  The cache row of a token is [latent | turned key part]."""
+    sliding window and (optionally) sink logits.  The cache row of a token is [latent | turned key
+    part]; a layer on another one's cache (``kv_from``) has only the query half of ``w_in``."""
 
     def __init__(self, spec, width: int):
         super().__init__()
@@ -122,29 +123,36 @@ class WindowLatentAttention(nn.Module):
     def set(self, dq, dq_norm, uq, dkv, dkv_norm, uk, uv, sink, o, dtype, device) -> None:
         s = self.spec
         H, D, Dr, V, R, Q, W = s.heads, s.dim, s.rot_dim, s.vdim, s.kv_rank, s.q_rank, self.width
-        assert Q > 0 and dq.shape == (Q, W) and uq.shape == (H * (D + Dr), Q) and dkv.shape == (R + Dr, W)
+        assert Q > 0 and dq.shape == (Q, W) and uq.shape == (H * (D + Dr), Q)
+        assert (dkv is None) == (s.kv_from >= 0) and (dkv is None or dkv.shape == (R + Dr, W))
         assert uk.shape == (H * D, R) and uv.shape == (H * V, R) and o.shape == (W, H * V)
         assert s.rot is None or (s.rot.dims % 2 == 0 and s.rot.dims <= Dr)
         to = lambda t: _p(t.to(device=device, dtype=dtype))
         f32 = lambda t: _p(t.to(device=device, dtype=torch.float32).reshape(-1))
-        self.w_in, self.uq, self.w_o = to(_pad_rows(torch.cat([dq, dkv], 0))), to(uq), to(o)
+        self.w_in = to(_pad_rows(dq if dkv is None else torch.cat([dq, dkv], 0)))
+        self.uq, self.w_o = to(uq), to(o)
         self.uk = to(uk.reshape(H, D, R))
         self.uv_t = to(uv.reshape(H, V, R).transpose(1, 2))
-        self.q_norm, self.kv_norm, self.sink = f32(dq_norm), f32(dkv_norm), f32(sink)
-        assert self.sink.numel() == H
+        self.q_norm, self.kv_norm = f32(dq_norm), f32(dkv_norm) if dkv is not None else None
+        assert (sink is not None) == s.sink
+        if s.sink:
+            self.sink = f32(sink)
+            assert self.sink.numel() == H
 
     def forward(self, h: torch.Tensor, positions: torch.Tensor, md, cache: tuple, eps: float):
         s = self.spec
         H, D, Dr, V, R = s.heads, s.dim, s.rot_dim, s.vdim, s.kv_rank
         T = h.shape[0]
+        halves = s.rot is None or s.rot.halves
+        own = s.kv_from < 0
         proj = _project(h, self.w_in, self.w_in_p)
-        cq = ma_ops.latent_in(proj[:, :s.q_rank + R + Dr], s.q_rank, R, Dr, self.q_norm, self.kv_norm, eps, positions, md.slot_mapping,
-                              self.table, True, cache[0])
+        cq = ma_ops.latent_in(proj[:, :s.q_rank + (R + Dr if own else 0)], s.q_rank, R, Dr, self.q_norm, self.kv_norm, eps,
+                              positions, md.slot_mapping, self.table, halves, cache[0] if own else None)
         q = _project(cq, self.uq, self.uq_p)
         q_lat = torch.bmm(q.view(T, H, D + Dr)[:, :, :D].transpose(0, 1), self.uk)                  # [H, T, R]
-        qf = ma_ops.latent_query(q_lat, q, D, Dr, positions, self.table, True)
+        qf = ma_ops.latent_query(q_lat, q, D, Dr, positions, self.table, halves)
         o_lat = ma_ops.masked_attention(qf, cache[0], None, R, md.block_tables, md.cu_q, md.context_lens, md.num_seqs,
-                                        s.scale, window=s.window, sink=self.sink if s.sink else None,
+                                        s.scale, window=s.window, sink=self.sink, fine=s.fine,
                                         out_dtype=h.dtype, head_major=True, num_decode=md.num_decode)                        # [H, T, R]
         o = torch.bmm(o_lat, self.uv_t).transpose(0, 1).reshape(T, H * V)
         return _project(o, self.w_o, self.w_o_p, partial=True)

@@ -39,11 +39,14 @@ class ExpertSum:
 
 
 def hyper_step(xs: torch.Tensor, y, close: Optional[tuple], open_: Optional[tuple], eps: float,
-               act_dtype: Optional[torch.dtype] = None, want_f32: bool = False, rows: Optional[torch.Tensor] = None):
+               act_dtype: Optional[torch.dtype] = None, want_f32: bool = False, rows: Optional[torch.Tensor] = None,
+               y_scale: Optional[torch.Tensor] = None, post_w: Optional[torch.Tensor] = None):
     """``close`` = (mix [S, S], a_out [S]) fp32: fold the sublayer output ``y`` ([T, W] tensor, the
     decode GEMM's unreduced split-K slabs, or an :class:`ExpertSum`) into the streams, in place.
+    ``y_scale`` [W] fp32: y is multiplied by it coordinate by coordinate first; ``post_w`` [W] fp32 (S = 1
+    only): y is first set to unit RMS times that weight.
     ``open_`` = (a_in [S], w [W]) fp32: z = u / sqrt(mean(u^2) + eps) * w of the (new) streams'
-    weighted sum u.  ``rows`` (only without ``close``): open these token rows only.
+    weighted sum u (w None: z = u).  ``rows`` (only without ``close``): open these token rows only.
     Returns (z in ``act_dtype`` or None, z in fp32 if ``want_f32`` else None)."""
     T, S, W = xs.shape
     assert xs.dtype == torch.float32 and xs.is_contiguous()
@@ -55,11 +58,15 @@ def hyper_step(xs: torch.Tensor, y, close: Optional[tuple], open_: Optional[tupl
         if close is not None:
             mix, a_out = close
             yv = y.total() if isinstance(y, ExpertSum) else y.float()
+            if post_w is not None:
+                yv = yv / torch.sqrt((yv * yv).mean(-1, keepdim=True) + eps) * post_w
+            if y_scale is not None:
+                yv = yv * y_scale
             xs.copy_(torch.einsum("st,nsw->ntw", mix, xs) + a_out[None, :, None] * yv[:, None, :])
         if open_ is not None:
             a_in, w = open_
             u = torch.einsum("s,nsw->nw", a_in, xs if rows is None else xs[rows.long()])
-            z = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * w
+            z = u if w is None else u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * w
             if act is not None:
                 act.copy_(z)
             if z32 is not None:
@@ -83,7 +90,7 @@ def hyper_step(xs: torch.Tensor, y, close: Optional[tuple], open_: Optional[tupl
                 native.ptr(es.gate) if es else None, es.gate.stride(0) if es and es.gate is not None else 0,
                 native.ptr(mix), native.ptr(a_out), native.ptr(a_in), native.ptr(w), float(eps), native.ptr(act),
                 native.dt_code(act_dtype) if act_dtype is not None else 1, native.ptr(z32), native.ptr(rows),
-                native.stream_ptr())
+                native.ptr(y_scale), native.ptr(post_w), native.stream_ptr())
     return act, z32
 
 
@@ -98,3 +105,16 @@ def spread_rows(table: torch.Tensor, ids: torch.Tensor, S: int, scale: float = 1
     native.call("pkm_spread_rows", xs.data_ptr(), table.data_ptr(), ids.data_ptr(), T, S, W, table.shape[0],
                 native.dt_code(table.dtype), float(scale), native.stream_ptr())
     return xs
+
+
+def embed_norm_rows(table: torch.Tensor, ids: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
+    """x[t] = table[ids[t]] set to unit RMS times w [W] fp32, as fp32 [T, 1, W] (one stream)."""
+    T, W = ids.numel(), table.shape[1]
+    if not table.is_cuda:
+        u = table[ids.long()].float()
+        return (u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * w)[:, None, :]
+    x = torch.empty((T, 1, W), dtype=torch.float32, device=table.device)
+    assert table.is_contiguous() and ids.dtype == torch.int32 and w.dtype == torch.float32 and w.numel() == W
+    native.call("pkm_embed_norm", x.data_ptr(), table.data_ptr(), ids.data_ptr(), w.data_ptr(), T, W, table.shape[0],
+                float(eps), native.dt_code(table.dtype), native.stream_ptr())
+    return x

@@ -9,9 +9,12 @@ state after the portion's last token.
 """
 from __future__ import annotations
 
+from typing import Optional
+
 import torch
 
 from . import native
+from .masked_attention import turn
 
 
 def lightning_attention(qkv: torch.Tensor, state: torch.Tensor, decay: torch.Tensor, cu_q: torch.Tensor,
@@ -42,6 +45,43 @@ def lightning_attention(qkv: torch.Tensor, state: torch.Tensor, decay: torch.Ten
     native.call("pkm_lightning_attention", out.data_ptr(), qkv.data_ptr(), qkv.stride(0), state.data_ptr(),
                 decay.data_ptr(), cu_q.data_ptr(), positions.data_ptr(), slots.data_ptr(), n_seqs, T, H, D, V,
                 int(num_decode), native.dt_code(qkv.dtype), native.stream_ptr())
+    return out
+
+
+def retention(qkv: torch.Tensor, state: torch.Tensor, decay: torch.Tensor, table: Optional[torch.Tensor], k_scale: float,
+              cu_q: torch.Tensor, n_seqs: int, positions: torch.Tensor, slots: torch.Tensor, H: int, D: int,
+              V: int) -> torch.Tensor:
+    """The same recurrence on plain projections: q and k turn by the token's position (``table``
+    [positions, pairs, 2] fp32 (cos, sin), pair i = (i, i + pairs); None: not) and k is multiplied by
+    ``k_scale``, both in fp32.  qkv [T, H*D | H*D | H*V] (may be a column slice) -> o [T, H * V] fp32."""
+    T = qkv.shape[0]
+    out = torch.empty((T, H * V), dtype=torch.float32, device=qkv.device)
+    if not qkv.is_cuda:
+        f = qkv.float()
+        q, k, v = f[:, :H * D].view(T, H, D), f[:, H * D:2 * H * D].view(T, H, D), f[:, 2 * H * D:].view(T, H, V)
+        if table is not None:
+            cs = table[positions.long()]
+            q, k = turn(q, cs), turn(k, cs)
+        k = k * k_scale
+        o3 = out.view(T, H, V)
+        for s in range(n_seqs):
+            a, b, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+            if b <= a:
+                continue
+            S = state[slot].clone() if (slot >= 0 and int(positions[a]) > 0) else torch.zeros((H, D, V))
+            for t in range(a, b):
+                S = decay[:, None, None] * S + k[t, :, :, None] * v[t, :, None, :]
+                o3[t] = torch.einsum("hdv,hd->hv", S, q[t])
+            if slot >= 0:
+                state[slot] = S
+        return out
+    assert qkv.stride(1) == 1 and state.is_contiguous() and state.dtype == torch.float32 and decay.dtype == torch.float32
+    assert state.shape[1:] == (H, D, V) and qkv.shape[1] == H * (2 * D + V) and decay.numel() == H
+    assert table is None or (table.dtype == torch.float32 and table.is_contiguous() and 2 * table.shape[1] <= D)
+    native.call("pkm_retention", out.data_ptr(), qkv.data_ptr(), qkv.stride(0), state.data_ptr(), decay.data_ptr(),
+                native.ptr(table), table.shape[1] if table is not None else 0, table.shape[0] if table is not None else 0,
+                float(k_scale), cu_q.data_ptr(), positions.data_ptr(), slots.data_ptr(), n_seqs, T, H, D, V,
+                native.dt_code(qkv.dtype), native.stream_ptr())
     return out
 
 

@@ -3,7 +3,9 @@ separate counts of query, key and value heads (csrc/mixers/masked_attention.hip;
 
 A query at position p sees keys j with lo(p) <= j <= p, where lo(p) = max(0, p - window + 1) for a
 sliding window (window > 0) and lo(p) = max(lo(p), floor(p / chunk) * chunk) for blocks of ``chunk``
-positions (chunk > 0); both 0: every earlier key.  The softmax denominator of query head h also
+positions (chunk > 0); both 0: every earlier key.  The first ``keep`` keys of the sequence may stay
+visible behind the band.  A table [QH, n] may add ``bias[h, min(p - j, n - 1)]`` to the scaled score
+(a learned distance bias).  The softmax denominator of query head h also
 holds exp(sink[h]) when sink logits are given (a key without a value).
 
 Query heads come in QH, key heads in KH, value heads in VH (QH % KH == 0, QH % VH == 0): query
@@ -45,6 +47,30 @@ def turn(x: torch.Tensor, cs: torch.Tensor, halves: bool = True) -> torch.Tensor
     return out
 
 
+def distance_bias(rel: torch.Tensor, bias_max: int) -> torch.Tensor:
+    """Learned bias by distance: rel [B, H] rows are buckets of the distance n between query and key, the
+    first h = B // 2 exact, the others evenly spaced in log n from h to ``bias_max`` (the last one holds
+    everything beyond).  Returns [H, n] fp32 indexed by min(distance, n - 1).  Bucket h + k starts
+    where n^m h^k >= h^m bias_max^k, m = B - h, compared in integers (no rounded logarithm)."""
+    B, H = rel.shape
+    h, m = B // 2, B - B // 2
+    row, n, k = [], 0, 0
+    while True:
+        if n < h:
+            row.append(n)
+        else:
+            if h > 0 and bias_max > h:
+                while k < m and n ** m * h ** (k + 1) >= h ** m * bias_max ** (k + 1):
+                    k += 1
+            else:
+                k = m
+            row.append(min(B - 1, h + k))
+        if row[-1] == B - 1:
+            break
+        n += 1
+    return rel.float()[row].t().contiguous()
+
+
 def _write_cache(cache: torch.Tensor, rows: torch.Tensor, slot_mapping: torch.Tensor) -> None:
     """cache [blocks, heads, bs, width] <- rows [T, heads, width] at the tokens' slots (< 0: not)."""
     bs = cache.shape[2]
@@ -56,11 +82,11 @@ def _write_cache(cache: torch.Tensor, rows: torch.Tensor, slot_mapping: torch.Te
 def rotate_cache(proj: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor, table: Optional[torch.Tensor],
                  halves: bool, k_cache: torch.Tensor, v_cache: torch.Tensor, QH: int, KH: int, VH: int, D: int,
                  V: int, q_norm: Optional[torch.Tensor] = None, k_norm: Optional[torch.Tensor] = None,
-                 eps: float = 0.0) -> torch.Tensor:
+                 eps: float = 0.0, v_unit: bool = False) -> torch.Tensor:
     """proj [T, QH*D | KH*D | VH*V] (may be a column slice of a wider projection output): q and k
     heads turn by the token's position (``table`` rows; None: no rotation), k and v go to the paged
     caches.  ``q_norm`` / ``k_norm`` [D] fp32: the heads are first set to unit RMS (``eps`` inside
-    the root) times that weight.  Returns q [T, QH, D] in the cache's dtype."""
+    the root) times that weight; ``v_unit``: each value head is set to unit RMS.  Returns q [T, QH, D] in the cache's dtype."""
     T = proj.shape[0]
     q = torch.empty((T, QH, D), dtype=k_cache.dtype, device=proj.device)
     if not proj.is_cuda:
@@ -72,6 +98,8 @@ def rotate_cache(proj: torch.Tensor, positions: torch.Tensor, slot_mapping: torc
             qq = unit(qq, q_norm)
         if k_norm is not None:
             kk = unit(kk, k_norm)
+        if v_unit:
+            vv = unit(vv, 1.0)
         if table is not None:
             cs = table[positions.long()]
             qq, kk = turn(qq, cs, halves), turn(kk, cs, halves)
@@ -89,7 +117,7 @@ def rotate_cache(proj: torch.Tensor, positions: torch.Tensor, slot_mapping: torc
     native.call("pkm_rotate_cache", q.data_ptr(), proj.data_ptr(), proj.stride(0), positions.data_ptr(),
                 slot_mapping.data_ptr(), native.ptr(table), table.shape[1] if table is not None else 0,
                 table.shape[0] if table is not None else 0, int(halves), k_cache.data_ptr(), v_cache.data_ptr(), T,
-                QH, KH, VH, D, V, k_cache.shape[2], native.ptr(q_norm), native.ptr(k_norm), float(eps),
+                QH, KH, VH, D, V, k_cache.shape[2], native.ptr(q_norm), native.ptr(k_norm), int(v_unit), float(eps),
                 native.dt_code(k_cache.dtype), native.stream_ptr())
     return q
 
@@ -97,21 +125,30 @@ def rotate_cache(proj: torch.Tensor, positions: torch.Tensor, slot_mapping: torc
 def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[torch.Tensor], V: int,
                      block_tables: torch.Tensor, cu_q: torch.Tensor, context_lens: torch.Tensor, n_seqs: int,
                      scale: float, window: int = 0, chunk: int = 0, sink: Optional[torch.Tensor] = None,
-                     out_dtype: torch.dtype = torch.float32, head_major: bool = False, num_decode: int = 0) -> torch.Tensor:
+                     out_dtype: torch.dtype = torch.float32, head_major: bool = False, num_decode: int = 0,
+                     keep: int = 0, bias: Optional[torch.Tensor] = None, post: float = 1.0, fine: bool = False,
+                     out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [T, QH, D] (fp32 or the cache's dtype); sequence s owns tokens cu_q[s]:cu_q[s+1], the LAST
     ones of its context_lens[s] cached tokens.  ``v_cache`` None: the value of a key is the first
     ``V`` numbers of its key row (key heads = value heads).  ``sink`` [QH] fp32 logits or None.
     The first ``num_decode`` sequences hold one token each (the matrix-core kernel cuts their bands
     into runs that a second kernel merges).  Returns [T, QH, V], or [QH, T, V] with ``head_major``,
-    in ``out_dtype``.  Scores, softmax and the value sums are fp32."""
+    in ``out_dtype``.  Scores, softmax and the value sums are fp32.  ``keep``: the first keys that stay
+    visible; ``bias`` [QH, n] fp32 (:func:`distance_bias`); ``post`` multiplies the result; ``fine``: the
+    matrix-core kernel sees the softmax weights to 16 bits (always with ``keep`` or ``bias``; a single
+    bf16 otherwise); ``out``: write there ([T, QH * V], may be a column slice of a wider row)."""
     T, QH, D = q.shape
     KH, bs = k_cache.shape[1], k_cache.shape[2]
     vc = k_cache if v_cache is None else v_cache
     VH = vc.shape[1]
-    out = torch.empty((QH, T, V) if head_major else (T, QH, V), dtype=out_dtype, device=q.device)
+    if out is None:
+        out = torch.empty((QH, T, V) if head_major else (T, QH, V), dtype=out_dtype, device=q.device)
+    else:
+        assert out.shape == (T, QH * V) and out.stride(1) == 1 and not head_major
+        out_dtype = out.dtype
     assert QH % KH == 0 and QH % VH == 0 and k_cache.shape[3] == D and V <= vc.shape[3]
     if not q.is_cuda:
-        o3 = out.transpose(0, 1) if head_major else out
+        o3 = out.transpose(0, 1) if head_major else out.unflatten(1, (QH, V)) if out.dim() == 2 else out
         for s in range(n_seqs):
             a, b, ctx = int(cu_q[s]), int(cu_q[s + 1]), int(context_lens[s])
             if b <= a:
@@ -127,7 +164,10 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[t
                 lo = torch.maximum(lo, pos - window + 1)
             if chunk > 0:
                 lo = torch.maximum(lo, pos // chunk * chunk)
-            seen = (idx[None, :] <= pos[:, None]) & (idx[None, :] >= lo[:, None])
+            back = pos[:, None] - idx[None, :]
+            seen = (back >= 0) & ((idx[None, :] >= lo[:, None]) | (idx[None, :] < keep))
+            if bias is not None:
+                sc = sc + bias[:, back.clamp(0, bias.shape[1] - 1)]
             sc = sc.masked_fill(~seen[None], float("-inf"))
             m = sc.amax(-1, keepdim=True)
             if sink is not None:
@@ -136,25 +176,27 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[t
             den = e.sum(-1, keepdim=True)
             if sink is not None:
                 den = den + torch.exp(sink[:, None, None] - m)
-            o3[a:b] = torch.einsum("htj,jhv->thv", e / den, v).to(out_dtype)
+            o3[a:b] = (torch.einsum("htj,jhv->thv", e / den, v) * post).to(out_dtype)
         return out
     assert q.is_contiguous() and k_cache.is_contiguous() and vc.is_contiguous() and vc.dtype == k_cache.dtype
     assert block_tables.stride(1) == 1 and (sink is None or (sink.dtype == torch.float32 and sink.numel() == QH))
     assert q.dtype in (torch.float32, k_cache.dtype)
-    ts, hs = (V, T * V) if head_major else (QH * V, V)
+    assert bias is None or (bias.dtype == torch.float32 and bias.is_contiguous() and bias.shape[0] == QH)
+    ts, hs = (V, T * V) if head_major else (out.stride(0), V)
     nd = min(num_decode, n_seqs)
     ws_o = ws_ml = None
     part = n_parts = 0
     if nd and q.dtype == k_cache.dtype:
         capacity = block_tables.shape[1] * bs
         part = native.mixers().pkm_masked_decode_part(nd, QH, KH, D, V, int(v_cache is None), bs, capacity, int(window),
-                                                      int(chunk), native.dt_code(k_cache.dtype))
+                                                      int(chunk), int(keep), native.dt_code(k_cache.dtype))
         if part > 0:
             span = capacity
             if window > 0:
                 span = min(span, window + 31)
             if chunk > 0:
                 span = min(span, chunk + 31)
+            span = min((span + 31) // 32 * 32 + (keep + 31) // 32 * 32, (capacity + 31) // 32 * 32)
             n_parts = -(-((span + 31) // 32 * 32) // part)
             if n_parts > 1:
                 ws_o = torch.empty((nd, n_parts, QH, V), dtype=torch.float32, device=q.device)
@@ -162,18 +204,19 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[t
     native.call("pkm_masked_attention", out.data_ptr(), ts, hs, native.dt_code(out_dtype), q.data_ptr(),
                 native.dt_code(q.dtype), k_cache.data_ptr(), vc.data_ptr(), vc.shape[3], block_tables.data_ptr(),
                 block_tables.stride(0), cu_q.data_ptr(), context_lens.data_ptr(), native.ptr(sink), n_seqs, T, QH, KH, VH,
-                D, V, bs, float(scale), int(window), int(chunk), nd, native.ptr(ws_o), native.ptr(ws_ml), part, n_parts,
+                D, V, bs, float(scale), int(window), int(chunk), int(keep), native.ptr(bias),
+                bias.shape[1] if bias is not None else 0, float(post), int(fine), nd, native.ptr(ws_o), native.ptr(ws_ml), part, n_parts,
                 native.dt_code(k_cache.dtype), native.stream_ptr())
     return out
 
 
 def latent_in(proj: torch.Tensor, q_rank: int, R: int, Dr: int, wq: Optional[torch.Tensor], wkv: torch.Tensor, eps: float,
               positions: torch.Tensor, slot_mapping: torch.Tensor, table: Optional[torch.Tensor], halves: bool,
-              cache: torch.Tensor) -> Optional[torch.Tensor]:
+              cache: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
     """proj [T, q_rank | R | Dr]: the query latent set to unit RMS times ``wq`` is returned
     ([T, q_rank], the projection's dtype; None with q_rank = 0); the key / value latent set to unit
     RMS times ``wkv`` and the shared key part turned by the position go to cache rows
-    [blocks, 1, block_size, R + Dr]."""
+    [blocks, 1, block_size, R + Dr].  ``cache`` None: ``proj`` is [T, q_rank], only the query latent is made."""
     T = proj.shape[0]
     cq = torch.empty((T, q_rank), dtype=proj.dtype, device=proj.device) if q_rank else None
     if not proj.is_cuda:
@@ -181,19 +224,26 @@ def latent_in(proj: torch.Tensor, q_rank: int, R: int, Dr: int, wq: Optional[tor
         unit = lambda t: t / torch.sqrt((t * t).mean(-1, keepdim=True) + eps)
         if q_rank:
             cq.copy_(unit(f[:, :q_rank]) * wq)
+        if cache is None:
+            return cq
         c = unit(f[:, q_rank:q_rank + R]) * wkv
         kr = f[:, q_rank + R:].view(T, 1, Dr)
         if table is not None and Dr:
             kr = turn(kr, table[positions.long()], halves)
         _write_cache(cache, torch.cat([c, kr[:, 0]], -1)[:, None, :], slot_mapping)
         return cq
-    assert proj.stride(1) == 1 and proj.shape[1] == q_rank + R + Dr and cache.is_contiguous() and cache.dtype == proj.dtype
-    assert cache.shape[1] == 1 and cache.shape[3] == R + Dr and wkv.dtype == torch.float32
+    if cache is None:
+        assert q_rank and proj.shape[1] == q_rank
+        R, Dr, wkv, table = 1, 0, None, None
+    else:
+        assert proj.shape[1] == q_rank + R + Dr and cache.is_contiguous() and cache.dtype == proj.dtype
+        assert cache.shape[1] == 1 and cache.shape[3] == R + Dr and wkv.dtype == torch.float32
+    assert proj.stride(1) == 1
     assert table is None or (table.dtype == torch.float32 and 2 * table.shape[1] <= Dr)
-    native.call("pkm_latent_in", native.ptr(cq), cache.data_ptr(), proj.data_ptr(), proj.stride(0), q_rank, R, Dr,
-                native.ptr(wq), wkv.data_ptr(), float(eps), positions.data_ptr(), slot_mapping.data_ptr(),
+    native.call("pkm_latent_in", native.ptr(cq), native.ptr(cache), proj.data_ptr(), proj.stride(0), q_rank, R, Dr,
+                native.ptr(wq), native.ptr(wkv), float(eps), positions.data_ptr(), slot_mapping.data_ptr(),
                 native.ptr(table), table.shape[1] if table is not None else 0, table.shape[0] if table is not None else 0,
-                int(halves), T, cache.shape[2], native.dt_code(proj.dtype), native.stream_ptr())
+                int(halves), T, cache.shape[2] if cache is not None else 1, native.dt_code(proj.dtype), native.stream_ptr())
     return cq
 
 

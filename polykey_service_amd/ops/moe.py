@@ -478,3 +478,101 @@ def silu_experts(x_act: torch.Tensor, ids: torch.Tensor, gate, up, down, w13=Non
                 offsets.data_ptr(), sorted_.data_ptr(), 0.0, n, k, E, F_, W, dt, st)
     native.call("pkm_expert_down", y.data_ptr(), h.data_ptr(), down.data_ptr(), offsets.data_ptr(), n, E, W, F_, dt, st)
     return y, inv
+
+
+# ------------------------------------------------------------------ group-limited routing, ungated experts, pointwise activations
+ACT_GELU, ACT_RELU2, ACT_XIELU = 0, 1, 2
+
+
+def route_group_topk(logits: torch.Tensor, correction: Optional[torch.Tensor], k: int, groups: int = 1,
+                     keep: int = 1) -> Tuple[torch.Tensor, torch.Tensor]:
+    """fp32 router logits [T, E] -> (ids [T, k] int32, weights [T, k]).  Scores are the softmax over all
+    experts; experts are chosen by score + ``correction`` [E] inside the ``keep`` best of ``groups`` equal
+    groups of neighbours (a group counts as its largest choice score), weighted by the score alone, not
+    renormalised.  Ties: the lower index."""
+    T, E = logits.shape
+    if not logits.is_cuda:
+        s = torch.softmax(logits.float(), -1)
+        c = s + correction if correction is not None else s.clone()
+        if groups > 1:
+            best = torch.sort(c.view(T, groups, -1).amax(-1), dim=-1, descending=True, stable=True).indices[:, :keep]
+            ok = torch.zeros((T, groups), dtype=torch.bool).scatter_(1, best, True)
+            c = c.masked_fill(~ok.repeat_interleave(E // groups, 1), float("-inf"))
+        ids = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :k]
+        return ids.to(torch.int32).contiguous(), s.gather(1, ids).contiguous()
+    assert logits.dtype == torch.float32 and logits.stride(1) == 1
+    assert correction is None or (correction.dtype == torch.float32 and correction.numel() == E)
+    ids = torch.empty((T, k), dtype=torch.int32, device=logits.device)
+    w = torch.empty((T, k), dtype=torch.float32, device=logits.device)
+    native.call("pkm_route_group_topk", ids.data_ptr(), w.data_ptr(), logits.data_ptr(), logits.stride(0),
+                native.ptr(correction), T, E, k, groups, keep, native.stream_ptr())
+    return ids, w
+
+
+def _act(z: torch.Tensor, kind: int, p: float, q: float) -> torch.Tensor:
+    if kind == ACT_RELU2:
+        return torch.relu(z) ** 2
+    if kind == ACT_XIELU:
+        return torch.where(z > 0, p * z * z, q * (torch.expm1(z) - z)) + 0.5 * z
+    return F.gelu(z, approximate="tanh")
+
+
+def activate(x, kind: int, p: float = 0.0, q: float = 0.0, dtype: Optional[torch.dtype] = None,
+             rows: Optional[tuple] = None) -> torch.Tensor:
+    """f(x) elementwise in fp32 maths: GELU (tanh form), max(x, 0)^2, or xIELU (p x^2 + x / 2 for x > 0,
+    q (exp(x) - 1 - x) + x / 2 otherwise).  x [n, N] is changed in place, or is a decode GEMM's
+    unreduced split-K slabs (``gemm.Partial``), summed on the way into a new tensor of ``dtype``.
+    ``rows`` = (table [vocab, R], ids [n] int32, off): also times table[ids[row], off + column]."""
+    part = isinstance(x, gemm.Partial)
+    n, N = (x.M, x.N) if part else x.shape
+    if not part and not x.is_cuda:
+        y = _act(x.float(), kind, p, q)
+        if rows is not None:
+            y = y * rows[0][rows[1].long(), rows[2]:rows[2] + N].float()
+        return x.copy_(y)
+    src = x.buf if part else x
+    out = torch.empty((n, N), dtype=dtype, device=src.device) if part else x
+    assert out.is_contiguous() and src.is_contiguous()
+    table, ids, off = rows if rows is not None else (None, None, 0)
+    assert table is None or (table.dtype == out.dtype and table.is_contiguous() and ids.dtype == torch.int32 and ids.numel() == n)
+    native.call("pkm_activate", out.data_ptr(), src.data_ptr(), x.S if part else 0, n, N, int(kind), float(p), float(q),
+                native.ptr(table), native.ptr(ids), table.shape[0] if table is not None else 0,
+                table.shape[1] if table is not None else 0, int(off), native.dt_code(out.dtype), native.stream_ptr())
+    return out
+
+
+def relu2_experts(x_act: torch.Tensor, ids: torch.Tensor, up, down, up_p=None, down_p=None, mfma: bool = False):
+    """Rows of every (token, chosen expert) pair through down_e(max(up_e x, 0)^2): (y [T * top, W] in expert
+    order, inv [T * top]).  up [E, F, W], down [E, W, F].  ``mfma`` (shapes of :func:`mfma_experts_ok`):
+    the framework's grouped MFMA GEMMs, else the tiled FMA grouped kernels (any sizes, fp32 too)."""
+    T, W = x_act.shape
+    k = ids.shape[1]
+    n = T * k
+    E, F_, _ = up.shape
+    offsets, sorted_, inv = align(ids, E, 0, E)
+    if mfma:
+        if T <= 64 and E <= 64 and gemm.SKINNY_ENABLED:  # decode: the GEMM gathers the tokens' rows itself
+            h = gemm.grouped_linear(x_act, up, offsets, T, False, packed=up_p, a_rows=sorted_, a_row_div=k, n_rows=n)
+            return gemm.grouped_linear(activate(h, ACT_RELU2), down, offsets, T, False, packed=down_p), inv
+        h = grouped_gemm(permute(x_act, sorted_, offsets, k), up, offsets, T, silu=False, packed=up_p)
+        return grouped_gemm(activate(h, ACT_RELU2), down, offsets, T, silu=False, packed=down_p), inv
+    if not x_act.is_cuda:
+        m = int(offsets[-1])
+        tok = sorted_[:m].long() // k
+        y = torch.zeros((m, W), dtype=torch.float32)
+        offs = offsets.tolist()
+        for e in range(E):
+            lo, hi = offs[e], offs[e + 1]
+            if hi > lo:
+                h = (torch.relu(F.linear(x_act[tok[lo:hi]], up[e]).float()) ** 2).to(x_act.dtype)
+                y[lo:hi] = F.linear(h, down[e]).float()
+        return y, inv
+    assert x_act.is_contiguous() and up.is_contiguous() and down.is_contiguous()
+    dt = native.dt_code(x_act.dtype)
+    h = torch.empty((n, F_), dtype=x_act.dtype, device=x_act.device)
+    y = torch.empty((n, W), dtype=torch.float32, device=x_act.device)
+    st = native.stream_ptr()
+    native.call("pkm_expert_up_relu2", h.data_ptr(), x_act.data_ptr(), up.data_ptr(), offsets.data_ptr(), sorted_.data_ptr(),
+                n, k, E, F_, W, dt, st)
+    native.call("pkm_expert_down", y.data_ptr(), h.data_ptr(), down.data_ptr(), offsets.data_ptr(), n, E, W, F_, dt, st)
+    return y, inv

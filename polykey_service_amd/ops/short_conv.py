@@ -24,11 +24,12 @@ ACT_NONE, ACT_SILU = 0, 1
 def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
                 cu_q: torch.Tensor, n_seqs: int, positions: torch.Tensor, slots: torch.Tensor, token_seq: torch.Tensor,
                 act: int = ACT_NONE, residual: bool = False, out_dtype: Optional[torch.dtype] = None,
-                in_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                in_bias: Optional[torch.Tensor] = None, num_decode: int = 0) -> torch.Tensor:
     """x [T, C] (may be a column slice of a wider row), taps [C, K] fp32, bias [C] fp32 or None.
     ``in_bias`` [C] fp32 is added to every input row first (a projection's bias: the filter and the
     state see x + in_bias, the zeros before the sequence stay zeros).  Returns [T, C] in
-    ``out_dtype`` (default: x's)."""
+    ``out_dtype`` (default: x's).  The first ``num_decode`` sequences hold one token each (all of them:
+    one kernel filters and moves the state)."""
     T, C = x.shape
     K = taps.shape[1]
     out = torch.empty((T, C), dtype=out_dtype or x.dtype, device=x.device)
@@ -61,5 +62,6 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor
     assert state is None or (state.dtype == torch.float32 and state.is_contiguous())
     native.call("pkm_causal_conv", out.data_ptr(), native.dt_code(out.dtype), x.data_ptr(), native.dt_code(x.dtype),
                 x.stride(0), native.ptr(in_bias), taps.data_ptr(), K, native.ptr(bias), native.ptr(state), cu_q.data_ptr(), positions.data_ptr(),
-                slots.data_ptr(), token_seq.data_ptr(), n_seqs, T, C, int(act), int(residual), native.stream_ptr())
+                slots.data_ptr(), token_seq.data_ptr(), n_seqs, T, C, int(act), int(residual), int(num_decode >= n_seqs),
+                native.stream_ptr())
     return out
