@@ -400,12 +400,12 @@ constexpr float kLog2e = 1.4426950408889634f;
 
 __host__ __device__ __forceinline__ int quad_slot(int q) { return (q & 3) * 8 + 4 * (q >> 2); }  // slot of key 4 q
 
-// FINE: the softmax weights enter the value product as two bf16 parts (16 bits of them), and the kept keys
-// and the distance bias are built in.
+// FINE: the softmax weights enter the value product as two bf16 parts (16 bits of them); where keys and
+// values are separate caches the kept keys and the distance bias are built in too.
 // SPLIT: one token per sequence; blockIdx.z picks a run of a.part of the walked keys and the
 // workgroup leaves (max, sum, unnormalised o) per row in the workspace (no sink: the merge adds it).
 template <int D, int V, int NW, bool ALIAS, bool SPLIT, bool FINE>
-__global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedArgs a) {
+__global__ void __launch_bounds__(64 * NW, (D <= 128 && V <= 128) ? 4 : 1) masked_attention_mfma_kernel(MaskedArgs a) {
   constexpr int NT = 64 * NW, BQ = 16 * NW, BK = 32, NKK = D / 32, NRT = V / 16, CS = D + 8, CT = BK + 8;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
   bf16_t* ks = reinterpret_cast<bf16_t*>(smem_raw);  // [BK][CS]  key-major
@@ -440,7 +440,8 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
   const int first_pos = ctx - qlen + row0 / R;
   const int max_pos = ctx - qlen + (min(row0 + BQ, n_rows) - 1) / R;
   const int k_begin = first_pos >= 0 ? first_key(first_pos, a.window, a.chunk) / BK * BK : 0;
-  const int keep = FINE ? a.keep : 0;
+  constexpr bool EXT = FINE && !ALIAS;
+  const int keep = EXT ? a.keep : 0;
   const int kept = kept_span(keep, k_begin, BK);
   // walked keys [w_begin, w_end): the kept tiles, then the band from its first tile
   int w_begin = 0, w_end = kept + max_pos + 1 - k_begin;
@@ -449,7 +450,7 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
     w_end = min(w_end, w_begin + a.part);
   }
   auto key_at = [&](int w) { return w < kept ? w : k_begin + w - kept; };
-  const float* my_bias = (FINE && a.bias) ? a.bias + static_cast<int64_t>(h) * a.bias_n : nullptr;
+  const float* my_bias = (EXT && a.bias) ? a.bias + static_cast<int64_t>(h) * a.bias_n : nullptr;
   const bf16_t* q = static_cast<const bf16_t*>(a.q);
   const bf16_t* kc = static_cast<const bf16_t*>(a.k_cache);
   const bf16_t* vc = static_cast<const bf16_t*>(a.v_cache);
@@ -476,6 +477,16 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
   constexpr int VUN = V;                   // units of (4 keys x 8 value columns): 8 quads x V / 8 column chunks
   constexpr int VIT = (VUN + NT - 1) / NT;
   pk::u32x4 kv[KIT], vv[VIT][4];
+  float bias[EXT ? 8 : 1];  // the tile's biases of this lane's scores, loaded one tile ahead
+  auto fetch_bias = [&](int k0) {
+    if (EXT && my_bias) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int back = my_pos - (k0 + (e >> 2) * 16 + 4 * g + (e & 3));
+        bias[e] = my_bias[min(max(back, 0), a.bias_n - 1)];
+      }
+    }
+  };
   auto fetch = [&](int k0) {
     const int64_t blk = bt[k0 / bs];
     const bf16_t* ksrc = kc + ((blk * KH + kh) * bs + k0 % bs) * D;
@@ -496,7 +507,10 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
       }
     }
   };
-  if (w_begin < w_end) fetch(key_at(w_begin));
+  if (w_begin < w_end) {
+    fetch_bias(key_at(w_begin));
+    fetch(key_at(w_begin));
+  }
   for (int w0 = w_begin; w0 < w_end; w0 += BK) {
     const int k0 = key_at(w0);
 #pragma unroll
@@ -528,14 +542,6 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
     __syncthreads();
     if (w0 + BK < w_end) fetch(key_at(w0 + BK));
     if (__any(my_pos >= k0 && (my_lo <= k0 + BK - 1 || k0 < keep))) {
-      float bias[8];
-      if (FINE && my_bias) {
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const int n_back = my_pos - (k0 + (e >> 2) * 16 + 4 * g + (e & 3));
-          bias[e] = my_bias[min(max(n_back, 0), a.bias_n - 1)] * kLog2e;
-        }
-      }
       pk::f32x4 sa[2] = {pk::f32x4{0.f, 0.f, 0.f, 0.f}, pk::f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
       for (int sub = 0; sub < 2; ++sub) {
@@ -550,7 +556,7 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
       for (int e = 0; e < 8; ++e) {
         const int key = k0 + (e >> 2) * 16 + 4 * g + (e & 3);
         float v = sa[e >> 2][e & 3] * sl2;
-        if (FINE && my_bias) v += bias[e];
+        if (EXT && my_bias) v += bias[e] * kLog2e;
         sc[e] = (key <= my_pos && (key >= my_lo || key < keep)) ? v : -INFINITY;
         tmax = fmaxf(tmax, sc[e]);
       }
@@ -577,20 +583,25 @@ __global__ void __launch_bounds__(64 * NW) masked_attention_mfma_kernel(MaskedAr
         for (int rt = 0; rt < NRT; ++rt) o[rt] *= resc;
       }
       const bf16_t* vr = vt + n * CT + 8 * g;
-#pragma unroll
-      for (int rt = 0; rt < NRT; ++rt)
-        o[rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pk::ld8(vr + rt * 16 * CT), pb, o[rt], 0, 0, 0);
-      if (FINE) {  // what rounding the weights to bf16 left over
-        pk::u32x4 lw;
+      if (FINE) {
+        pk::u32x4 lw;  // what rounding the weights to bf16 left over
 #pragma unroll
         for (int e = 0; e < 4; ++e)
           lw[e] = pk::pack2(p[2 * e] - __uint_as_float(pw[e] << 16), p[2 * e + 1] - __uint_as_float(pw[e] & 0xffff0000u));
         const pk::bf16x8_t lb = __builtin_bit_cast(pk::bf16x8_t, lw);
 #pragma unroll
+        for (int rt = 0; rt < NRT; ++rt) {
+          const pk::bf16x8_t va = pk::ld8(vr + rt * 16 * CT);
+          o[rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, pb, o[rt], 0, 0, 0);
+          o[rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, lb, o[rt], 0, 0, 0);
+        }
+      } else {
+#pragma unroll
         for (int rt = 0; rt < NRT; ++rt)
-          o[rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pk::ld8(vr + rt * 16 * CT), lb, o[rt], 0, 0, 0);
+          o[rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pk::ld8(vr + rt * 16 * CT), pb, o[rt], 0, 0, 0);
       }
     }
+    if (w0 + BK < w_end) fetch_bias(key_at(w0 + BK));
     __syncthreads();
   }
   if (SPLIT) {
@@ -817,7 +828,7 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
   const bool finer = fine || keep > 0 || bias;
   const int R = QH / KH;
   if (g_masked_mfma && dt == kBF16 && q_dt == kBF16 && bs % 32 == 0 && v_width % 8 == 0 && out_ts % 4 == 0 && out_hs % 4 == 0 &&
-      mfma_sizes(D, V, alias)) {
+      mfma_sizes(D, V, alias) && !(alias && (keep > 0 || bias))) {
     // the first num_decode sequences hold one token each: their bands are cut into runs when a
     // workspace is given (ws_o [num_decode, n_parts, QH, V], ws_ml [num_decode, n_parts, QH, 2] fp32)
     const int nd = (ws_o && ws_ml && n_parts > 1) ? (num_decode < n_seqs ? num_decode : n_seqs) : 0;
