@@ -701,10 +701,10 @@ int launch_mfma(const MaskedArgs& a, int T, bool alias, hipStream_t stream) {
   if (a.D == DD && a.V == VV && alias == AL) return launch_mfma_one<DD, VV, (SPLIT ? NWS : NW), AL, SPLIT, FINE>(a, T, stream);
   // waves per workgroup for prompt portions / for decoded tokens (one 16-row tile computes there:
   // fewer, less loaded waves stage the tiles faster for the wide rows)
-  PKM_MM(64, 64, 8, 8, false)
-  PKM_MM(64, 128, 8, 8, false)
-  PKM_MM(128, 64, 8, 8, false)
-  PKM_MM(128, 128, 8, 8, false)
+  PKM_MM(64, 64, 8, 4, false)
+  PKM_MM(64, 128, 8, 4, false)
+  PKM_MM(128, 64, 8, 4, false)
+  PKM_MM(128, 128, 8, 4, false)
   PKM_MM(96, 64, 8, 8, true)
   PKM_MM(160, 128, 8, 8, true)
   PKM_MM(192, 128, 8, 8, true)
@@ -869,7 +869,7 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
 
 // Keys per run of a decoded token's band (a multiple of 32), 0: no split.  `capacity`: the most
 // cached tokens of a sequence; the band spans at most window + 31 / chunk + 31 keys from its
-// aligned start, with the kept keys' tiles in front.  Runs are at least 64 keys, at most 64 of them, and aim at ~512 workgroups per launch.
+// aligned start, with the kept keys' tiles in front.  Runs are at least 64 keys, at most 64 of them, and aim at 512 or 1024 workgroups per launch.
 PK_EXPORT int pkm_masked_decode_part(int nd, int QH, int KH, int D, int V, int alias, int bs, int capacity, int window,
                                      int chunk, int keep, int dt) {
   if (!g_masked_mfma || dt != kBF16 || bs % 32 || nd <= 0 || !mfma_sizes(D, V, alias != 0)) return 0;
@@ -879,7 +879,9 @@ PK_EXPORT int pkm_masked_decode_part(int nd, int QH, int KH, int D, int V, int a
   span = (span + 31) / 32 * 32 + (keep + 31) / 32 * 32;
   if (span > (capacity + 31) / 32 * 32) span = (capacity + 31) / 32 * 32;
   const int wgs = nd * KH;
-  int want = (512 + wgs - 1) / wgs;  // runs wanted
+  // narrow heads: four workgroups of four waves fit a CU; wide latent rows: two
+  const int fill = (D <= 128 && V <= 128) ? 1024 : 512;
+  int want = (fill + wgs - 1) / wgs;  // runs wanted
   if (want > 64) want = 64;
   if (want > span / 64) want = span / 64;
   if (want <= 1) return 0;

@@ -465,18 +465,18 @@ class LefuvikForCausalLM(nn.Module):
             raise RuntimeError("Lefuvik: reserve_positions(max_model_len) has not been called")
         close = (self.unit_mix, self.one)
 
-        def step(y, open_w, **kw):
-            return hyper_ops.hyper_step(x, y, close if y is not None else None, (self.one, open_w), eps, dt, **kw)
+        def step(y, open_, **kw):
+            return hyper_ops.hyper_step(x, y, close if y is not None else None, open_, eps, dt, **kw)
         x = hyper_ops.embed_norm_rows(self.embed, input_ids, self.embed_norm, eps)
-        h, _ = step(None, self.layers[0].norm1)
+        h, _ = step(None, (self.one, self.layers[0].norm1))
         for i, L in enumerate(self.layers):
-            nxt = self.layers[i + 1].norm1 if i + 1 < len(self.layers) else self.final_norm
+            nxt = (self.one, self.layers[i + 1].norm1) if i + 1 < len(self.layers) else None
             y, scale = L.mix(h, positions, md, caches[i], eps), L.scale1
             if L.mlp is not None:
-                h, h32 = step(y, L.norm2, y_scale=scale, want_f32=isinstance(L.mlp, GroupedMoE))
+                h, h32 = step(y, (self.one, L.norm2), y_scale=scale, want_f32=isinstance(L.mlp, GroupedMoE))
                 y, scale = L.mlp(h, h32), L.scale2
             if L.side is not None:
-                xa, _ = step(y, None, y_scale=scale)
+                xa, _ = step(y, (self.one, None), y_scale=scale)
                 h, _ = step(L.side(xa, self.side_embed, input_ids), nxt, post_w=L.side.norm_w)
             else:
                 h, _ = step(y, nxt, y_scale=scale)
