@@ -40,14 +40,13 @@ def softplus(z):
 
 def rotate(x, dims, base, interleaved):
     """x [T, heads, d]: the first ``dims`` coordinates of every head turn by position * base^(-2i/dims)."""
-    out = x.clone()
-    for p in range(x.shape[0]):
-        for i in range(dims // 2):
-            a = p * base ** (-2.0 * i / dims)
-            iu, iv = (2 * i, 2 * i + 1) if interleaved else (i, i + dims // 2)
-            u, v = x[p, :, iu], x[p, :, iv]
-            out[p, :, iu] = u * math.cos(a) - v * math.sin(a)
-            out[p, :, iv] = v * math.cos(a) + u * math.sin(a)
+    out, p = x.clone(), torch.arange(x.shape[0], dtype=D64)
+    for i in range(dims // 2):
+        a = (p * base ** (-2.0 * i / dims))[:, None]
+        iu, iv = (2 * i, 2 * i + 1) if interleaved else (i, i + dims // 2)
+        u, v = x[:, :, iu], x[:, :, iv]
+        out[:, :, iu] = u * torch.cos(a) - v * torch.sin(a)
+        out[:, :, iv] = v * torch.cos(a) + u * torch.sin(a)
     return out
 
 
@@ -252,7 +251,7 @@ def forward(cfg, w, tokens):
 
 
 # ------------------------------------------------------------------ small random models
-def random_model(cfg, seed=0, std=None, dtype=torch.bfloat16):
+def random_model(cfg, seed=0, std=None, dtype=torch.bfloat16, buckets=8):
     """Random weights (representable in ``dtype``) under the checkpoint's names."""
     g = torch.Generator().manual_seed(seed)
     W, w = cfg["width"], {}
@@ -273,7 +272,7 @@ def random_model(cfg, seed=0, std=None, dtype=torch.bfloat16):
             lin(q1 + "q", a["heads"] * a["dim"], W), lin(q1 + "k", a["kv_heads"] * a["dim"], W)
             lin(q1 + "v", a["kv_heads"] * a["vdim"], W), lin(q1 + "o", W, a["heads"] * a["vdim"])
             r(q1 + "q.norm", (a["dim"],), 0.3, 1.0), r(q1 + "k.norm", (a["dim"],), 0.3, 1.0)
-            r(q1 + "rel", (l.get("buckets", 8), a["heads"]), 1.0)
+            r(q1 + "rel", (buckets, a["heads"]), 1.0)
             C, nb = b["width"], b["blocks"]
             for n in "yx":
                 lin(q2 + n, C, W), r(q2 + n + ".b", (C,), 0.3)
@@ -305,3 +304,42 @@ def random_model(cfg, seed=0, std=None, dtype=torch.bfloat16):
             d = cfg["token_side"]["dim"]
             lin(p + "side.gate", d, W), lin(p + "side.proj", W, d), r(p + "side.norm", (W,), 0.2, 0.5)
     return w
+
+
+def make_config(pattern=("parallel:dense", "retention:moe", "latent:moe", "parallel:none", "shared:moe"), vocab=61, width=40, heads=4,
+                kv_heads=2, dim=12, vdim=8, window=21, keep=6, bias_max=30, rwidth=36, blocks=3, conv=4, left=0.7, right=1.2,
+                rheads=3, rdim=10, rvdim=14, rrot=6, lheads=2, ldim=9, lvdim=11, kv_rank=20, q_rank=26, rot_dim=8, lwindow=18,
+                ff=52, experts=6, top=2, eff=24, groups=3, keep_groups=2, side=5, cap=12.0, eps=1e-5):
+    """A small configuration: ``pattern`` lists mixer:feed-forward ("shared" is latent attention on the
+    last "latent" layer's cache)."""
+    layers, last = [], None
+    for i, item in enumerate(pattern):
+        kind, f = item.split(":")
+        if kind == "parallel":
+            mask = {"size": window, "keep_first": keep}
+            m = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": 1.3 * dim ** -0.5,
+                          "bias_max": bias_max, "mask": mask},
+                 "right": {"width": rwidth, "blocks": blocks, "conv": conv}, "left_scale": left, "right_scale": right}
+        elif kind == "retention":
+            m = {"heads": rheads, "dim": rdim, "vdim": rvdim, "decay": [1 - 2.0 ** (-2 - 2 * h) for h in range(rheads)],
+                 "rot": {"dims": rrot, "base": 700.0}}
+        else:
+            m = {"heads": lheads, "dim": ldim, "vdim": lvdim, "kv_rank": kv_rank, "q_rank": q_rank, "rot_dim": rot_dim,
+                 "scale": 1.1 * (ldim + rot_dim) ** -0.5, "rot": {"dims": rot_dim, "base": 300.0}, "mask": {"size": lwindow}}
+            if kind == "shared":
+                m["kv_from"] = last
+                m["mask"] = {"size": lwindow + 7}
+            else:
+                last = i
+        mlp = None
+        if f == "dense":
+            mlp = {"kind": "dense", "ff": ff}
+        elif f == "moe":
+            mlp = {"kind": "moe", "expert": {"ff": eff}, "router": {"experts": experts, "top": top}}
+            if groups > 1:
+                mlp["router"]["groups"] = {"count": groups, "keep": keep_groups}
+        layers.append({"type": {"latent": "latent_attention", "shared": "latent_attention"}.get(kind, kind), "mixer": m, "mlp": mlp})
+    cfg = {"architecture": "Lefuvik", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers, "logit_softcap": cap}
+    if side:
+        cfg["token_side"] = {"dim": side}
+    return cfg
