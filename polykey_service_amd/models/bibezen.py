@@ -156,7 +156,7 @@ class SelectiveScanMixer(nn.Module):
         seq = (md.cu_q, md.num_seqs, positions, md.state_slots)
         xz = _project(h, self.w_in, self.w_in_p)
         x = conv_ops.causal_conv(xz[:, :I], self.taps, self.conv_b, cache.get("conv"), *seq, md.token_seq,
-                                 act=conv_ops.ACT_SILU)
+                                 act=conv_ops.ACT_SILU, num_decode=md.num_decode)
         low = gemm.linear(x, self.w_x)
         d = gemm.linear(low[:, :R].contiguous(), self.w_dt)
         y = scan_ops.selective_scan(x, d, self.dt_b, self.A, low[:, R:], self.D, xz[:, I:2 * I], cache["scan"], *seq)
@@ -228,7 +228,7 @@ class ParallelMixer(nn.Module):
         a = torch.empty((T, self.w_o.shape[1]), dtype=h.dtype, device=h.device)
         proj = _project(h, self.w_in, self.w_in_p)
         qkv = conv_ops.causal_conv(proj[:, :C], self.taps, None, cache.get("conv"), md.cu_q, md.num_seqs, positions,
-                                   md.state_slots, md.token_seq, in_bias=self.bias)
+                                   md.state_slots, md.token_seq, in_bias=self.bias, num_decode=md.num_decode)
         kc, vc = cache["k"], cache["v"]
         q = ma_ops.rotate_cache(qkv, positions, md.slot_mapping, self.table, True, kc, vc, H, G, G, D, V,
                                 q_norm=self.q_norm, k_norm=self.k_norm, eps=eps)
@@ -588,7 +588,7 @@ class BibezenForCausalLM(nn.Module):
             cache = caches[i]
             if L.canon is not None:
                 h = conv_ops.causal_conv(h, L.canon, None, cache.get("canon"), md.cu_q, md.num_seqs, positions,
-                                         md.state_slots, md.token_seq, residual=True)
+                                         md.state_slots, md.token_seq, residual=True, num_decode=md.num_decode)
             y = L.mix(h, positions, md, cache, eps)
             close = L.hc1[1:]
             if L.mlp is not None:
