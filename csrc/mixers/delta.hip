@@ -6,6 +6,7 @@
 //                by sqrt(D)); a second kernel brings the slot's last K - 1 inputs up to date
 //   delta_rule   per (sequence, head), token by token, S [D, V] fp32:
 //                  gate = exp(-exp(A_log_h) softplus(a + dt_bias_h)),  beta = sigmoid(b)
+//                  (or one gate per key channel d, made by conv_unit's launch: row d of S times gate_d)
 //                  S <- gate S ;  u = beta (v - S^T k) ;  S <- S + k u^T ;  o = S^T q
 //
 // The state of a (sequence, head) lives in the sequence's state slot between steps.  In delta_rule a
@@ -24,14 +25,33 @@ __device__ __forceinline__ float softplusf(float z) { return fmaxf(z, 0.f) + log
 
 constexpr int kMaxTaps = 64;  // the kernels loop over the taps; this only bounds a wrong argument
 
-// one wave per (token, head): heads 0..G-1 q, G..2G-1 k, then H value heads
+// per-channel decays of the recurrence: gates[t, h, d] = exp(-exp(a_log_h) softplus(z[t, h, d] + dt_bias[h, d]))
+struct ChannelDecay {
+  float* gates;  // [T, H, D] or null
+  const void* z; // the projections' element type, rows `stride` elements apart
+  int64_t stride;
+  const float* a_log;
+  const float* dt_bias;
+};
+
+// one wave per (token, head): heads 0..G-1 q, G..2G-1 k, then H value heads, then (cd.gates) H heads' decays.
+// single: every sequence holds one token; a lane then moves its channels' slot rows itself.
 template <typename T>
 __global__ void __launch_bounds__(64)
 conv_unit_kernel(float* __restrict__ out, const T* __restrict__ proj, int64_t stride, const float* __restrict__ taps, int K,
-                 const float* __restrict__ conv_state, const int* __restrict__ cu_q, const int* __restrict__ positions,
-                 const int* __restrict__ slots, const int* __restrict__ token_seq, int G, int D, int H, int V) {
+                 float* __restrict__ conv_state, const int* __restrict__ cu_q, const int* __restrict__ positions,
+                 const int* __restrict__ slots, const int* __restrict__ token_seq, int G, int D, int H, int V,
+                 ChannelDecay cd, int single) {
   const int t = blockIdx.x, item = blockIdx.y, lane = threadIdx.x;
   const int C = 2 * G * D + H * V;
+  if (item >= 2 * G + H) {  // one head's decays
+    const int h = item - 2 * G - H;
+    const T* z = static_cast<const T*>(cd.z) + static_cast<int64_t>(t) * cd.stride + static_cast<int64_t>(h) * D;
+    const float rate = -expf(cd.a_log[h]);
+    float* g = cd.gates + (static_cast<int64_t>(t) * H + h) * D;
+    for (int d = lane; d < D; d += 64) g[d] = expf(rate * softplusf(ld<T>(z + d) + cd.dt_bias[h * D + d]));
+    return;
+  }
   const bool qk = item < 2 * G;
   const int width = qk ? D : V;
   const int c0 = qk ? item * D : 2 * G * D + (item - 2 * G) * V;
@@ -39,7 +59,7 @@ conv_unit_kernel(float* __restrict__ out, const T* __restrict__ proj, int64_t st
   const int a = cu_q[s], slot = slots[s];
   const int i = t - a;  // index inside the portion
   const bool carry = slot >= 0 && positions[a] > 0;
-  const float* past = conv_state + static_cast<int64_t>(slot < 0 ? 0 : slot) * (K > 1 ? K - 1 : 1) * C;
+  float* past = conv_state + static_cast<int64_t>(slot < 0 ? 0 : slot) * (K > 1 ? K - 1 : 1) * C;
   float ss = 0.f;
   for (int d0 = 0; d0 < width; d0 += 64) {
     const int d = d0 + lane;
@@ -54,6 +74,7 @@ conv_unit_kernel(float* __restrict__ out, const T* __restrict__ proj, int64_t st
         } else if (carry) {
           x = past[static_cast<int64_t>(K - 1 + rel) * C + c];
         }
+        if (single && slot >= 0 && j > 0) past[static_cast<int64_t>(j - 1) * C + c] = x;  // row j was read before
         y += taps[static_cast<int64_t>(c) * K + j] * x;
       }
       y = siluf(y);
@@ -107,10 +128,12 @@ __device__ __forceinline__ float quad_sum(float v) {
 // k of a token lie in LDS as 4 runs of ND (+ 4 floats of padding, so the quad's four 16-byte reads
 // fall on different banks).  The next group's q, k, v are fetched into registers before the
 // current group is computed.
-template <typename AT, int ND>
+// CH: one gate per key channel, read from gates [T, H, D] and staged like q and k; ab is then b alone.
+template <typename AT, int ND, bool CH>
 __global__ void __launch_bounds__(256)
 delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const AT* __restrict__ ab, int64_t ab_stride,
-                  const float* __restrict__ a_log, const float* __restrict__ dt_bias, float* __restrict__ state,
+                  const float* __restrict__ a_log, const float* __restrict__ dt_bias, const float* __restrict__ gates,
+                  float* __restrict__ state,
                   const int* __restrict__ cu_q, const int* __restrict__ positions, const int* __restrict__ slots, int G, int D,
                   int H, int V, int kChunk) {
   constexpr int RS = ND + 4, TS = 4 * RS;          // floats per run and per token
@@ -118,7 +141,8 @@ delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
   extern __shared__ __attribute__((aligned(16))) float smem[];
   float* qs = smem;                 // [kChunk][4][RS]
   float* ks = qs + kChunk * TS;     // [kChunk][4][RS]
-  float* vs = ks + kChunk * TS;     // [kChunk][kCols]
+  float* cs = ks + kChunk * TS;     // [kChunk][4][RS] (CH)
+  float* vs = CH ? cs + kChunk * TS : cs;  // [kChunk][kCols]
   float* gs = vs + kChunk * kCols;  // [kChunk] gate
   float* bs_ = gs + kChunk;         // [kChunk] beta
   const int s = blockIdx.x / H, h = blockIdx.x - s * H;
@@ -130,7 +154,7 @@ delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
   const int C = 2 * G * D + H * V;
   const int nd = (D + 3) / 4;
   const int kvh = h / (H / G);
-  const float neg_rate = -expf(a_log[h]), bias = dt_bias[h];
+  const float neg_rate = CH ? 0.f : -expf(a_log[h]), bias = CH ? 0.f : dt_bias[h];
   float* sp = slot >= 0 ? state + ((static_cast<int64_t>(slot) * H + h) * D) * V : nullptr;
   const bool carry = sp != nullptr && positions[a] > 0;
   float S[ND];
@@ -141,7 +165,7 @@ delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
   }
   const int64_t qo = static_cast<int64_t>(kvh) * D, ko = static_cast<int64_t>(G + kvh) * D;
   const int64_t vo = 2 * static_cast<int64_t>(G) * D + static_cast<int64_t>(h) * V + v0;
-  float rq[QK_IT], rk[QK_IT], rv[V_IT];
+  float rq[QK_IT], rk[QK_IT], rc[CH ? QK_IT : 1], rv[V_IT];
   auto fetch = [&](int t0) {  // the group starting at token t0 (zeros outside the head's D rows)
     const int nt = min(kChunk, b - t0);
 #pragma unroll
@@ -152,6 +176,7 @@ delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
       const float* row = qkv + static_cast<int64_t>(t0 + (ok ? t : 0)) * C;
       rq[i] = ok ? row[qo + d] : 0.f;
       rk[i] = ok ? row[ko + d] : 0.f;
+      if (CH) rc[i] = ok ? gates[(static_cast<int64_t>(t0 + t) * H + h) * D + d] : 0.f;
     }
 #pragma unroll
     for (int i = 0; i < V_IT; ++i) {
@@ -170,6 +195,7 @@ delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
       if (t < kChunk) {
         qs[t * TS + su * RS + ii] = rq[i];
         ks[t * TS + su * RS + ii] = rk[i];
+        if (CH) cs[t * TS + su * RS + ii] = rc[i];
       }
     }
 #pragma unroll
@@ -179,16 +205,27 @@ delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
     }
     if (tid < nt) {
       const AT* r = ab + static_cast<int64_t>(t0 + tid) * ab_stride;
-      gs[tid] = expf(neg_rate * softplusf(ld<AT>(r + h) + bias));
-      bs_[tid] = sigmoidf(ld<AT>(r + H + h));
+      if (!CH) gs[tid] = expf(neg_rate * softplusf(ld<AT>(r + h) + bias));
+      bs_[tid] = sigmoidf(ld<AT>(r + (CH ? 0 : H) + h));
     }
     __syncthreads();
     if (t0 + kChunk < b) fetch(t0 + kChunk);  // in flight while this group is computed
     for (int t = 0; t < nt; ++t) {
-      const float gate = gs[t], beta = bs_[t];
+      const float gate = CH ? 1.f : gs[t], beta = bs_[t];
       const float vv = vs[t * kCols + (tid >> 2)];
       const float4* kr = reinterpret_cast<const float4*>(ks + t * TS + sub * RS);
       const float4* qr = reinterpret_cast<const float4*>(qs + t * TS + sub * RS);
+      if (CH) {  // the rows decay first
+        const float4* cr = reinterpret_cast<const float4*>(cs + t * TS + sub * RS);
+#pragma unroll
+        for (int i = 0; i < ND / 4; ++i) {
+          const float4 c4 = cr[i];
+          S[4 * i] *= c4.x;
+          S[4 * i + 1] *= c4.y;
+          S[4 * i + 2] *= c4.z;
+          S[4 * i + 3] *= c4.w;
+        }
+      }
       float r0 = 0.f, r1 = 0.f, r2 = 0.f, r3 = 0.f;
 #pragma unroll
       for (int i = 0; i < ND / 4; ++i) {
@@ -229,21 +266,27 @@ delta_rule_kernel(float* __restrict__ out, const float* __restrict__ qkv, const 
 }  // namespace
 
 // out fp32 [T, C], C = 2 G D + H V; proj [T, C] rows `stride` elements apart; taps [C, K] fp32;
-// conv_state [slots, K - 1, C] fp32 (read, then brought up to date by a second launch)
+// conv_state [slots, K - 1, C] fp32 (read, then brought up to date by a second launch; with `single`, where
+// every sequence holds one token, by the same one); gates fp32 [T, H, D] or null: per-channel decays from z
+// [T, H*D] (element type dt, rows z_stride apart), a_log [H], dt_bias [H*D] fp32
 PK_EXPORT int pkm_conv_unit(void* out, const void* proj, long long stride, const void* taps, int K, void* conv_state,
                             const void* cu_q, const void* positions, const void* slots, const void* token_seq, int n_seqs,
-                            int T, int G, int D, int H, int V, int dt, hipStream_t stream) {
+                            int T, int G, int D, int H, int V, void* gates, const void* z, long long z_stride,
+                            const void* a_log, const void* dt_bias, int single, int dt, hipStream_t stream) {
   if (T <= 0 || n_seqs <= 0) return 0;
   if (K < 1 || K > kMaxTaps || G < 1 || H < 1 || D < 1 || V < 1) return -1;
+  if (gates && (!z || !a_log || !dt_bias || z_stride < static_cast<long long>(H) * D)) return -1;
+  if (single && n_seqs != T) return -1;
   const int C = 2 * G * D + H * V;
-  const dim3 grid(T, 2 * G + H);
+  const ChannelDecay cd{static_cast<float*>(gates), z, z_stride, static_cast<const float*>(a_log), static_cast<const float*>(dt_bias)};
+  const dim3 grid(T, 2 * G + H + (gates ? H : 0));
   PKM_DISPATCH(dt, E, conv_unit_kernel<E><<<grid, 64, 0, stream>>>(
                           static_cast<float*>(out), static_cast<const E*>(proj), stride, static_cast<const float*>(taps), K,
-                          static_cast<const float*>(conv_state), static_cast<const int*>(cu_q),
+                          static_cast<float*>(conv_state), static_cast<const int*>(cu_q),
                           static_cast<const int*>(positions), static_cast<const int*>(slots),
-                          static_cast<const int*>(token_seq), G, D, H, V));
+                          static_cast<const int*>(token_seq), G, D, H, V, cd, single));
   int rc = PK_CHECK_LAUNCH();
-  if (rc || K == 1) return rc;
+  if (rc || K == 1 || single) return rc;
   const dim3 sgrid((C + 255) / 256, n_seqs);
   PKM_DISPATCH(dt, E, conv_state_kernel<E><<<sgrid, 256, 0, stream>>>(
                           static_cast<float*>(conv_state), static_cast<const E*>(proj), stride, K,
@@ -253,24 +296,31 @@ PK_EXPORT int pkm_conv_unit(void* out, const void* proj, long long stride, const
 }
 
 // out [T, H, V] fp32; qkv fp32 [T, G*D | G*D | H*V]; ab [T, H | H] rows ab_stride elements apart
-// (ab_dt); state [slots, H, D, V] fp32
+// (ab_dt); state [slots, H, D, V] fp32.  gates fp32 [T, H, D]: one gate per key channel; ab is then b [T, H] and
+// a_log, dt_bias are null
 PK_EXPORT int pkm_delta_rule(void* out, const void* qkv, const void* ab, long long ab_stride, int ab_dt, const void* a_log,
-                             const void* dt_bias, void* state, const void* cu_q, const void* positions, const void* slots,
-                             int n_seqs, int T, int G, int D, int H, int V, hipStream_t stream) {
+                             const void* dt_bias, const void* gates, void* state, const void* cu_q, const void* positions,
+                             const void* slots, int n_seqs, int T, int G, int D, int H, int V, hipStream_t stream) {
   if (n_seqs <= 0 || T <= 0) return 0;
-  if (D < 1 || D > 512 || V < 1 || G < 1 || H % G) return -1;
+  if (D < 1 || D > 512 || V < 1 || G < 1 || H % G || (!gates && (!a_log || !dt_bias))) return -1;
   const dim3 grid(n_seqs * H, (V + kCols - 1) / kCols);
   const int nd = (D + 3) / 4;
   const int ndt = nd <= 8 ? 8 : nd <= 16 ? 16 : nd <= 32 ? 32 : nd <= 64 ? 64 : 128;
-  const int per_tok = 8 * (ndt + 4) + kCols + 2;  // floats of LDS per staged token
+  const int per_tok = (gates ? 12 : 8) * (ndt + 4) + kCols + 2;  // floats of LDS per staged token
   const int chunk = max(1, min(kMaxChunk, 15360 / per_tok));  // at most 60 KiB of LDS
   const size_t lds = static_cast<size_t>(chunk) * per_tok * sizeof(float);
-#define PKM_DELTA(ND)                                                                                                 \
-  PKM_DISPATCH(ab_dt, E, delta_rule_kernel<E, ND><<<grid, 256, lds, stream>>>(                                          \
+#define PKM_DELTA_CH(ND, CH)                                                                                           \
+  PKM_DISPATCH(ab_dt, E, delta_rule_kernel<E, ND, CH><<<grid, 256, lds, stream>>>(                                     \
                              static_cast<float*>(out), static_cast<const float*>(qkv), static_cast<const E*>(ab), ab_stride, \
                              static_cast<const float*>(a_log), static_cast<const float*>(dt_bias),                     \
-                             static_cast<float*>(state), static_cast<const int*>(cu_q), static_cast<const int*>(positions), \
-                             static_cast<const int*>(slots), G, D, H, V, chunk))
+                             static_cast<const float*>(gates), static_cast<float*>(state), static_cast<const int*>(cu_q), \
+                             static_cast<const int*>(positions), static_cast<const int*>(slots), G, D, H, V, chunk))
+#define PKM_DELTA(ND)        \
+  if (gates) {               \
+    PKM_DELTA_CH(ND, true);  \
+  } else {                   \
+    PKM_DELTA_CH(ND, false); \
+  }
   if (nd <= 8) {
     PKM_DELTA(8);
   } else if (nd <= 16) {
@@ -283,5 +333,6 @@ PK_EXPORT int pkm_delta_rule(void* out, const void* qkv, const void* ab, long lo
     PKM_DELTA(128);
   }
 #undef PKM_DELTA
+#undef PKM_DELTA_CH
   return PK_CHECK_LAUNCH();
 }

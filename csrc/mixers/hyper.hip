@@ -10,6 +10,8 @@
 //                 coordinate (y_scale); without a norm weight the opened sum u itself is z.
 //                 Either half may be absent; with `rows` only those tokens are opened (the rows whose
 //                 logits are wanted).  S = 1 with unit coefficients is the plain residual.
+//   pair_step     closes a sublayer of two branches on one stream: y = ca U(ya) wa + cb U(yb) wb,
+//                 x <- x + U(y) post_w, act = x, U(u) = u / sqrt(mean(u^2) + eps); slabs summed on the way
 //   embed_norm    x[t] = table[ids[t]] set to unit RMS times a weight, as fp32
 //   tanh_cap      x <- cap * tanh(x / cap)
 //
@@ -272,6 +274,96 @@ __global__ void __launch_bounds__(1024) hyper_step_kernel(HyperArgs a) {
   }
 }
 
+struct PairArgs {
+  float* x;
+  int W;
+  const void* y[2];
+  int nslab[2];
+  int64_t slab_stride;
+  const float* w[2];
+  float c[2];
+  const float* post_w;
+  float eps;
+  void* act;
+};
+
+// NG >= 1: W % 4 == 0, a thread owns up to NG groups of four coordinates of both branches in registers;
+// NG = 0: any W, one coordinate at a time through LDS.
+template <typename T, typename Y, int NG>
+__global__ void __launch_bounds__(1024) pair_step_kernel(PairArgs a) {
+  __shared__ float red[16];
+  extern __shared__ __attribute__((aligned(16))) float vbuf[];  // [2][W] (NG = 0)
+  const int64_t r = blockIdx.x;
+  const int W = a.W;
+  float* x = a.x + r * W;
+  T* act = static_cast<T*>(a.act) + r * W;
+  const float inv_w = 1.f / static_cast<float>(W);
+  if (NG > 0) {
+    constexpr int N = NG > 0 ? NG : 1;
+    float4 v[2][N];
+    float ss[2] = {0.f, 0.f};
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      const Y* y = static_cast<const Y*>(a.y[b]) + r * W;
+#pragma unroll
+      for (int it = 0; it < N; ++it) {
+        const int i = 4 * (threadIdx.x + it * blockDim.x);
+        if (i >= W) break;
+        float4 u = ld4<Y>(y + i);
+        for (int sl = 1; sl < a.nslab[b]; ++sl) u = fma4(1.f, ld4<Y>(y + sl * a.slab_stride + i), u);
+        v[b][it] = u;
+        ss[b] += (u.x * u.x + u.y * u.y) + (u.z * u.z + u.w * u.w);
+      }
+    }
+    const float k0 = a.c[0] / sqrtf(pk::block_sum(ss[0], red) * inv_w + a.eps);
+    const float k1 = a.c[1] / sqrtf(pk::block_sum(ss[1], red) * inv_w + a.eps);
+    float sy = 0.f;
+#pragma unroll
+    for (int it = 0; it < N; ++it) {
+      const int i = 4 * (threadIdx.x + it * blockDim.x);
+      if (i >= W) break;
+      const float4 y0 = mul4(v[0][it], ld4<float>(a.w[0] + i)), y1 = mul4(v[1][it], ld4<float>(a.w[1] + i));
+      const float4 u = fma4(k0, y0, float4{k1 * y1.x, k1 * y1.y, k1 * y1.z, k1 * y1.w});
+      v[0][it] = u;
+      sy += (u.x * u.x + u.y * u.y) + (u.z * u.z + u.w * u.w);
+    }
+    const float k = 1.f / sqrtf(pk::block_sum(sy, red) * inv_w + a.eps);
+#pragma unroll
+    for (int it = 0; it < N; ++it) {
+      const int i = 4 * (threadIdx.x + it * blockDim.x);
+      if (i >= W) break;
+      const float4 z = fma4(k, mul4(v[0][it], ld4<float>(a.post_w + i)), ld4<float>(x + i));
+      st4<float>(x + i, z);
+      st4<T>(act + i, z);
+    }
+    return;
+  }
+  float ss[2] = {0.f, 0.f};
+  for (int b = 0; b < 2; ++b) {
+    const Y* y = static_cast<const Y*>(a.y[b]) + r * W;
+    for (int i = threadIdx.x; i < W; i += blockDim.x) {
+      float u = ld<Y>(y + i);
+      for (int sl = 1; sl < a.nslab[b]; ++sl) u += ld<Y>(y + sl * a.slab_stride + i);
+      vbuf[b * W + i] = u;  // read back by this thread only
+      ss[b] += u * u;
+    }
+  }
+  const float k0 = a.c[0] / sqrtf(pk::block_sum(ss[0], red) * inv_w + a.eps);
+  const float k1 = a.c[1] / sqrtf(pk::block_sum(ss[1], red) * inv_w + a.eps);
+  float sy = 0.f;
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float u = k0 * vbuf[i] * a.w[0][i] + k1 * vbuf[W + i] * a.w[1][i];
+    vbuf[i] = u;
+    sy += u * u;
+  }
+  const float k = 1.f / sqrtf(pk::block_sum(sy, red) * inv_w + a.eps);
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float z = x[i] + k * vbuf[i] * a.post_w[i];
+    x[i] = z;
+    st<T>(act + i, z);
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) embed_norm_kernel(float* __restrict__ x, const T* __restrict__ table,
                                                          const int* __restrict__ ids, const float* __restrict__ w, int W,
@@ -395,6 +487,57 @@ PK_EXPORT int pkm_hyper_step(void* xs, int R, int S, int W, const void* y, int y
     }
 #undef PKM_HS1
   }
+  return PK_CHECK_LAUNCH();
+}
+
+// x [R, W] fp32, updated in place; ya / yb: [R, W] rows (nslab > 1: fp32 slabs [nslab][R][W]) of one element type; wa, wb,
+// post_w [W] fp32; act [R, W] of type act_dt takes the new rows
+PK_EXPORT int pkm_pair_step(void* x, int R, int W, const void* ya, int na, int ya_dt, const void* yb, int nb, int yb_dt,
+                            const void* wa, const void* wb, float ca, float cb, const void* post_w, float eps, void* act,
+                            int act_dt, hipStream_t stream) {
+  if (R <= 0) return 0;
+  if (W < 1 || W > 16384 || na < 1 || nb < 1 || !ya || !yb || !wa || !wb || !post_w || !act || ya_dt != yb_dt) return -1;
+  if (ya_dt != kF32 && (ya_dt != kBF16 || na > 1 || nb > 1)) return -2;
+  const PairArgs a{static_cast<float*>(x), W, {ya, yb}, {na, nb}, static_cast<int64_t>(R) * W,
+                   {static_cast<const float*>(wa), static_cast<const float*>(wb)}, {ca, cb}, static_cast<const float*>(post_w), eps, act};
+#define PKM_PS(NG, THREADS, LDS)                                                                    \
+  if (ya_dt == kF32) {                                                                              \
+    PKM_DISPATCH(act_dt, E, pair_step_kernel<E, float, NG><<<R, THREADS, LDS, stream>>>(a));        \
+  } else {                                                                                          \
+    PKM_DISPATCH(act_dt, E, pair_step_kernel<E, bf16_t, NG><<<R, THREADS, LDS, stream>>>(a));       \
+  }
+  if (W % 4) {
+    const size_t lds = 2 * static_cast<size_t>(W) * sizeof(float);
+    const int threads = W >= 4096 ? 1024 : 256;
+    if (lds > 60 * 1024) {
+      const void* kern = nullptr;
+      if (ya_dt == kF32) {
+        kern = act_dt == kF32 ? reinterpret_cast<const void*>(pair_step_kernel<float, float, 0>)
+                              : reinterpret_cast<const void*>(pair_step_kernel<bf16_t, float, 0>);
+      } else {
+        kern = act_dt == kF32 ? reinterpret_cast<const void*>(pair_step_kernel<float, bf16_t, 0>)
+                              : reinterpret_cast<const void*>(pair_step_kernel<bf16_t, bf16_t, 0>);
+      }
+      const hipError_t e = hipFuncSetAttribute(kern, hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds));
+      if (e != hipSuccess) return static_cast<int>(e);
+    }
+    PKM_PS(0, threads, lds)
+    return PK_CHECK_LAUNCH();
+  }
+  // prompt-sized launches: up to four groups per thread (few waves per token, many tokens per CU); decode-sized
+  // ones: one group per thread
+  const int groups = W / 4;
+  int threads = ((R > 1024 ? (groups + 3) / 4 : groups) + 63) / 64 * 64;
+  threads = threads > 1024 ? 1024 : threads;
+  const int per = (groups + threads - 1) / threads;
+  if (per <= 1) {
+    PKM_PS(1, threads, 0)
+  } else if (per <= 2) {
+    PKM_PS(2, threads, 0)
+  } else {
+    PKM_PS(4, threads, 0)
+  }
+#undef PKM_PS
   return PK_CHECK_LAUNCH();
 }
 

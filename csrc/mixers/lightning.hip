@@ -4,6 +4,8 @@
 //
 // Retention is the same recurrence on plain projections (no SiLU): q and k turn by the token's
 // position in fp32 (pair (i, i + pairs), (cos, sin) table rows) and k is multiplied by k_scale.
+// The step form (state-space duality) has a step size d = softplus(dt + bias) per (token, head): decay
+// exp(-exp(a_log_h) d), v scaled by d on its way in, k / q shared by groups of heads, skip_h v added to o.
 // The state S [D, V] of a (sequence, head) is fp32 and lives in the sequence's state slot between
 // steps.  One workgroup owns 16 value columns of one (sequence, head): thread (dg, vc) keeps rows
 // dg, dg + 16, ... of column vc in registers and walks the portion's tokens in order; q, k, v of up to
@@ -26,7 +28,39 @@ struct HeadIn {
   int pairs, rows;
   const int* positions;
   float k_scale;
+  // step form: rows of the input are [H*V v | G*D k | G*D q]
+  const void* dt;        // [T, H] pre-activations, rows dt_stride apart
+  int64_t dt_stride;
+  int groups;
+  const float* dt_bias;  // [H] each
+  const float* a_log;
+  const float* skip;
 };
+
+enum Form { kSilu, kTurned, kStep };
+
+struct HeadAt {
+  int64_t q, k, v;  // first columns of a head in the input row
+};
+
+template <Form F>
+__device__ __forceinline__ HeadAt head_at(const HeadIn& in, int h, int H, int D, int V) {
+  if (F == kStep) {
+    const int64_t g = h / (H / in.groups), k0 = static_cast<int64_t>(H) * V;
+    return HeadAt{k0 + (in.groups + g) * D, k0 + g * D, static_cast<int64_t>(h) * V};
+  }
+  const int64_t q = static_cast<int64_t>(h) * D, hd = static_cast<int64_t>(H) * D;
+  return HeadAt{q, hd + q, 2 * hd + static_cast<int64_t>(h) * V};
+}
+
+__device__ __forceinline__ float softplusf(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+
+// step size and decay of (token t, head h)
+template <typename T>
+__device__ __forceinline__ void step_at(const HeadIn& in, int64_t t, int h, float& d, float& dec) {
+  d = softplusf(ld<T>(static_cast<const T*>(in.dt) + t * in.dt_stride + h) + in.dt_bias[h]);
+  dec = expf(-expf(in.a_log[h]) * d);
+}
 
 __device__ __forceinline__ float siluf(float z) { return z / (1.f + expf(-z)); }
 
@@ -43,7 +77,7 @@ __device__ __forceinline__ float turned(const T* src, int d, int64_t t, const He
   return first ? x * cs[0] - y * cs[1] : x * cs[0] + y * cs[1];
 }
 
-template <typename T, int ND, bool RET>
+template <typename T, int ND, Form F>
 __global__ void __launch_bounds__(256)
 lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t stride, float* __restrict__ state,
                  const float* __restrict__ decay, const int* __restrict__ cu_q, const int* __restrict__ positions,
@@ -52,6 +86,7 @@ lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t str
   float* qs = smem;                 // [kChunk][D]
   float* ks = qs + kChunk * D;      // [kChunk][D]
   float* vs = ks + kChunk * D;      // [kChunk][kCols]
+  float* ds = vs + kChunk * kCols;  // [kChunk][2] step size, decay (kStep)
   const int s = blockIdx.x / H, h = blockIdx.x - s * H;
   const int v0 = blockIdx.y * kCols;
   const int a = cu_q[s], b = cu_q[s + 1];
@@ -59,7 +94,7 @@ lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t str
   const int tid = threadIdx.x, dg = tid & 15, vc = tid >> 4;
   const int col = v0 + vc;
   const int slot = slots[s];
-  const float dec = decay[h];
+  const float dec_h = F == kStep ? 0.f : decay[h], skip = F == kStep ? in.skip[h] : 0.f;
   float S[ND];
   float* sp = slot >= 0 ? state + ((static_cast<int64_t>(slot) * H + h) * D) * V : nullptr;
   const bool carry = sp != nullptr && positions[a] > 0;
@@ -68,25 +103,33 @@ lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t str
     const int d = dg + 16 * i;
     S[i] = (carry && d < D && col < V) ? sp[static_cast<int64_t>(d) * V + col] : 0.f;
   }
-  const int64_t qo = static_cast<int64_t>(h) * D, ko = static_cast<int64_t>(H) * D + qo;
-  const int64_t vo = 2 * static_cast<int64_t>(H) * D + static_cast<int64_t>(h) * V + v0;
+  const HeadAt at = head_at<F>(in, h, H, D, V);
+  const int64_t qo = at.q, ko = at.k, vo = at.v + v0;
   for (int t0 = a; t0 < b; t0 += kChunk) {
     const int nt = min(kChunk, b - t0);
     __syncthreads();
     for (int e = tid; e < nt * D; e += 256) {
       const int t = e / D, d = e - t * D;
       const T* row = qkv + static_cast<int64_t>(t0 + t) * stride;
-      qs[e] = RET ? turned(row + qo, d, t0 + t, in) : siluf(ld<T>(row + qo + d));
-      ks[e] = RET ? turned(row + ko, d, t0 + t, in) * in.k_scale : siluf(ld<T>(row + ko + d));
+      if (F == kTurned) {
+        qs[e] = turned(row + qo, d, t0 + t, in);
+        ks[e] = turned(row + ko, d, t0 + t, in) * in.k_scale;
+      } else {
+        const float q = ld<T>(row + qo + d), k = ld<T>(row + ko + d);
+        qs[e] = F == kSilu ? siluf(q) : q;
+        ks[e] = F == kSilu ? siluf(k) : k;
+      }
     }
     for (int e = tid; e < nt * kCols; e += 256) {
       const int t = e / kCols, c = e - t * kCols;
       const float v = v0 + c < V ? ld<T>(qkv + static_cast<int64_t>(t0 + t) * stride + vo + c) : 0.f;
-      vs[e] = RET ? v : siluf(v);
+      vs[e] = F == kSilu ? siluf(v) : v;
     }
+    if (F == kStep && tid < nt) step_at<T>(in, t0 + tid, h, ds[2 * tid], ds[2 * tid + 1]);
     __syncthreads();
     for (int t = 0; t < nt; ++t) {
-      const float vv = vs[t * kCols + vc];
+      const float dec = F == kStep ? ds[2 * t + 1] : dec_h;
+      const float vv = F == kStep ? ds[2 * t] * vs[t * kCols + vc] : vs[t * kCols + vc];
       const float* kr = ks + t * D;
       const float* qr = qs + t * D;
       float o = 0.f;
@@ -102,6 +145,7 @@ lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t str
       o += __shfl_xor(o, 4, 64);
       o += __shfl_xor(o, 2, 64);
       o += __shfl_xor(o, 1, 64);
+      if (F == kStep) o += skip * vs[t * kCols + vc];
       if (dg == 0 && col < V) out[(static_cast<int64_t>(t0 + t) * H + h) * V + col] = o;
     }
   }
@@ -123,7 +167,7 @@ lightning_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t str
 constexpr int kWideChunk = 16;
 constexpr int kWideCols = 64;
 
-template <typename T, int NR, int NW, bool RET>
+template <typename T, int NR, int NW, Form F>
 __global__ void __launch_bounds__(64 * NW)
 lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_t stride, float* __restrict__ state,
                       const float* __restrict__ decay, const int* __restrict__ cu_q, const int* __restrict__ positions,
@@ -135,6 +179,7 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
   __shared__ __attribute__((aligned(16))) float ks[kWideChunk][DP];
   __shared__ float vs[kWideChunk][kWideCols];
   __shared__ float po[NW][kWideChunk][kWideCols];
+  __shared__ float ds[F == kStep ? kWideChunk : 1][2];  // step size, decay
   const int s = blockIdx.x / H, h = blockIdx.x - s * H;
   const int v0 = blockIdx.y * kWideCols;
   const int a = cu_q[s], b = cu_q[s + 1];
@@ -142,7 +187,7 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   const int col = v0 + lane;
   const int slot = slots[s];
-  const float dec = decay[h];
+  const float dec_h = F == kStep ? 0.f : decay[h], skip = F == kStep ? in.skip[h] : 0.f;
   float* sp = slot >= 0 ? state + ((static_cast<int64_t>(slot) * H + h) * D) * V : nullptr;
   const bool carry = sp != nullptr && positions[a] > 0;
   float S[NR];
@@ -151,8 +196,8 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
     const int d = w * NR + i;
     S[i] = (carry && d < D && col < V) ? sp[static_cast<int64_t>(d) * V + col] : 0.f;
   }
-  const int64_t qo = static_cast<int64_t>(h) * D, ko = static_cast<int64_t>(H) * D + qo;
-  const int64_t vo = 2 * static_cast<int64_t>(H) * D + static_cast<int64_t>(h) * V + v0;
+  const HeadAt at = head_at<F>(in, h, H, D, V);
+  const int64_t qo = at.q, ko = at.k, vo = at.v + v0;
   float rq[QK_IT], rk[QK_IT], rv[V_IT];
   auto fetch = [&](int t0) {  // raw projections of the group starting at token t0 (zeros outside)
     const int nt = min(kWideChunk, b - t0);
@@ -161,19 +206,19 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
       const int e = tid + NT * i, t = e / DP, d = e - t * DP;
       const bool ok = t < nt && d < D;
       const T* row = qkv + static_cast<int64_t>(t0 + (ok ? t : 0)) * stride;
-      if (RET) {
+      if (F == kTurned) {
         rq[i] = ok ? turned(row + qo, d, t0 + t, in) : 0.f;
         rk[i] = ok ? turned(row + ko, d, t0 + t, in) * in.k_scale : 0.f;
       } else {
-        rq[i] = ok ? ld<T>(row + qo + d) : -INFINITY;
-        rk[i] = ok ? ld<T>(row + ko + d) : -INFINITY;
+        rq[i] = ok ? ld<T>(row + qo + d) : (F == kSilu ? -INFINITY : 0.f);
+        rk[i] = ok ? ld<T>(row + ko + d) : (F == kSilu ? -INFINITY : 0.f);
       }
     }
 #pragma unroll
     for (int i = 0; i < V_IT; ++i) {
       const int e = tid + NT * i, t = e / kWideCols, c = e - t * kWideCols;
       const bool ok = t < nt && v0 + c < V;
-      rv[i] = ok ? ld<T>(qkv + static_cast<int64_t>(t0 + (ok ? t : 0)) * stride + vo + c) : (RET ? 0.f : -INFINITY);
+      rv[i] = ok ? ld<T>(qkv + static_cast<int64_t>(t0 + (ok ? t : 0)) * stride + vo + c) : (F == kSilu ? -INFINITY : 0.f);
     }
   };
   fetch(a);
@@ -183,23 +228,25 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
     for (int i = 0; i < QK_IT; ++i) {
       const int e = tid + NT * i;
       if (e < kWideChunk * DP) {
-        (&qs[0][0])[e] = RET ? rq[i] : (rq[i] == -INFINITY ? 0.f : siluf(rq[i]));
-        (&ks[0][0])[e] = RET ? rk[i] : (rk[i] == -INFINITY ? 0.f : siluf(rk[i]));
+        (&qs[0][0])[e] = F != kSilu ? rq[i] : (rq[i] == -INFINITY ? 0.f : siluf(rq[i]));
+        (&ks[0][0])[e] = F != kSilu ? rk[i] : (rk[i] == -INFINITY ? 0.f : siluf(rk[i]));
       }
     }
 #pragma unroll
     for (int i = 0; i < V_IT; ++i) {
       const int e = tid + NT * i;
-      if (e < kWideChunk * kWideCols) (&vs[0][0])[e] = RET ? rv[i] : (rv[i] == -INFINITY ? 0.f : siluf(rv[i]));
+      if (e < kWideChunk * kWideCols) (&vs[0][0])[e] = F != kSilu ? rv[i] : (rv[i] == -INFINITY ? 0.f : siluf(rv[i]));
     }
+    if (F == kStep && tid < nt) step_at<T>(in, t0 + tid, h, ds[tid][0], ds[tid][1]);
     __syncthreads();
     if (t0 + kWideChunk < b) fetch(t0 + kWideChunk);  // in flight while this group is computed
 #pragma unroll 4
     for (int t = 0; t < nt; ++t) {
-      const float vv = vs[t][lane];
+      const float dec = F == kStep ? ds[t][1] : dec_h;
+      const float vv = F == kStep ? ds[t][0] * vs[t][lane] : vs[t][lane];
       const float* kr = &ks[t][w * NR];
       const float* qr = &qs[t][w * NR];
-      float o0 = 0.f, o1 = 0.f;
+      float o0 = (F == kStep && w == 0) ? skip * vs[t][lane] : 0.f, o1 = 0.f;
       if (NR % 4 == 0) {
 #pragma unroll
         for (int i = 0; i < NR; i += 4) {
@@ -236,7 +283,7 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
         out[(static_cast<int64_t>(t0 + t) * H + h) * V + v0 + c] = o;
       }
     }
-    // the next group's staging writes qs / ks / vs only; po is rewritten after its barrier
+    // the next group's staging writes qs / ks / vs / ds only; po is rewritten after its barrier
   }
   if (sp != nullptr && col < V) {
 #pragma unroll
@@ -251,7 +298,7 @@ lightning_wide_kernel(float* __restrict__ out, const T* __restrict__ qkv, int64_
 
 namespace {
 
-template <bool RET>
+template <Form F>
 int launch_linear(void* out, const void* qkv, long long stride, void* state, const void* decay, const void* cu_q,
                   const void* positions, const void* slots, int n_seqs, int H, int D, int V, int dt, const HeadIn& in,
                   hipStream_t stream) {
@@ -260,7 +307,7 @@ int launch_linear(void* out, const void* qkv, long long stride, void* state, con
     const int nw = D > 64 ? 8 : 4;
     const int nr = (D + nw - 1) / nw;
 #define PKM_LIGHTW(NR, NW)                                                                                          \
-  PKM_DISPATCH(dt, E, lightning_wide_kernel<E, NR, NW, RET><<<wgrid, 64 * NW, 0, stream>>>(                          \
+  PKM_DISPATCH(dt, E, lightning_wide_kernel<E, NR, NW, F><<<wgrid, 64 * NW, 0, stream>>>(                          \
                           static_cast<float*>(out), static_cast<const E*>(qkv), stride, static_cast<float*>(state), \
                           static_cast<const float*>(decay), static_cast<const int*>(cu_q),                          \
                           static_cast<const int*>(positions), static_cast<const int*>(slots), H, D, V, in))
@@ -287,10 +334,10 @@ int launch_linear(void* out, const void* qkv, long long stride, void* state, con
     return PK_CHECK_LAUNCH();
   }
   const dim3 grid(n_seqs * H, (V + kCols - 1) / kCols);
-  const int chunk = max(1, min(kMaxChunk, 15360 / (2 * D + kCols)));  // at most 60 KiB of LDS
-  const size_t lds = static_cast<size_t>(chunk) * (2 * D + kCols) * sizeof(float);
+  const int chunk = max(1, min(kMaxChunk, 15360 / (2 * D + kCols + 2)));  // at most 60 KiB of LDS
+  const size_t lds = static_cast<size_t>(chunk) * (2 * D + kCols + 2) * sizeof(float);
   // heads of more than 256 key coordinates (narrower ones took the wider form)
-  PKM_DISPATCH(dt, E, lightning_kernel<E, 32, RET><<<grid, 256, lds, stream>>>(
+  PKM_DISPATCH(dt, E, lightning_kernel<E, 32, F><<<grid, 256, lds, stream>>>(
                           static_cast<float*>(out), static_cast<const E*>(qkv), stride, static_cast<float*>(state),
                           static_cast<const float*>(decay), static_cast<const int*>(cu_q),
                           static_cast<const int*>(positions), static_cast<const int*>(slots), H, D, V, chunk, in));
@@ -306,8 +353,8 @@ PK_EXPORT int pkm_lightning_attention(void* out, const void* qkv, long long stri
                                       int H, int D, int V, int num_decode, int dt, hipStream_t stream) {
   if (n_seqs <= 0 || T <= 0) return 0;
   if (D < 1 || D > 512 || V < 1) return -1;
-  return launch_linear<false>(out, qkv, stride, state, decay, cu_q, positions, slots, n_seqs, H, D, V, dt,
-                              HeadIn{nullptr, 0, 0, nullptr, 1.f}, stream);
+  return launch_linear<kSilu>(out, qkv, stride, state, decay, cu_q, positions, slots, n_seqs, H, D, V, dt,
+                              HeadIn{nullptr, 0, 0, nullptr, 1.f, nullptr, 0, 1, nullptr, nullptr, nullptr}, stream);
 }
 
 // the recurrence on plain projections: q and k turned by the position (table [rows, pairs, 2] fp32 or null), k
@@ -318,7 +365,23 @@ PK_EXPORT int pkm_retention(void* out, const void* qkv, long long stride, void* 
                             hipStream_t stream) {
   if (n_seqs <= 0 || T <= 0) return 0;
   if (D < 1 || D > 512 || V < 1 || 2 * pairs > D || (table && (rows < 1 || pairs < 1))) return -1;
-  return launch_linear<true>(out, qkv, stride, state, decay, cu_q, positions, slots, n_seqs, H, D, V, dt,
-                             HeadIn{static_cast<const float*>(table), pairs, rows, static_cast<const int*>(positions), k_scale},
+  return launch_linear<kTurned>(out, qkv, stride, state, decay, cu_q, positions, slots, n_seqs, H, D, V, dt,
+                             HeadIn{static_cast<const float*>(table), pairs, rows, static_cast<const int*>(positions), k_scale,
+                                    nullptr, 0, 1, nullptr, nullptr, nullptr},
                              stream);
+}
+
+// the step form: out [T, H, V] fp32; xbc [T, H*V | G*N | G*N] rows `stride` elements apart; dt [T, H] of the same element
+// type, rows dt_stride apart; dt_bias, a_log, skip [H] fp32; state [slots, H, N, V] fp32
+PK_EXPORT int pkm_step_scan(void* out, const void* xbc, long long stride, const void* dt, long long dt_stride, int G,
+                            const void* dt_bias, const void* a_log, const void* skip, void* state, const void* cu_q,
+                            const void* positions, const void* slots, int n_seqs, int T, int H, int N, int V, int dtype,
+                            hipStream_t stream) {
+  if (n_seqs <= 0 || T <= 0) return 0;
+  if (N < 1 || N > 512 || V < 1 || G < 1 || H < 1 || H % G || !dt || !dt_bias || !a_log || !skip) return -1;
+  if (stride < static_cast<long long>(H) * V + 2ll * G * N || dt_stride < H) return -1;
+  return launch_linear<kStep>(out, xbc, stride, state, nullptr, cu_q, positions, slots, n_seqs, H, N, V, dtype,
+                              HeadIn{nullptr, 0, 0, nullptr, 1.f, dt, dt_stride, G, static_cast<const float*>(dt_bias),
+                                     static_cast<const float*>(a_log), static_cast<const float*>(skip)},
+                              stream);
 }

@@ -3,7 +3,8 @@
 // the per-head norm / gate behind it.
 //
 //   rotate_cache      q and k heads turn by the token's position (fp32 (cos, sin) table rows; pair i
-//                     = (i, i + pairs) or (2i, 2i + 1)); q -> [T, QH, D], k -> cache
+//                     = (i, i + pairs) or (2i, 2i + 1)), q optionally times a factor that grows with the
+//                     position's logarithm; q -> [T, QH, D], k -> cache
 //                     [blocks, KH, block_size, D], v -> cache [blocks, VH, block_size, V]
 //   latent_in         a projection row [query latent | key / value latent | shared key part]: both
 //                     latents set to unit RMS times a weight, the key part turned by the position;
@@ -13,7 +14,7 @@
 //                     floor(p / chunk) chunk); p_j = exp(s_j) / (exp(sink_h) + sum_j' exp(s_j')),
 //                     s = q . k * scale; o = sum_j p_j v_j.  The first `keep` keys may stay visible behind
 //                     the band (j < keep, j <= p); a table may add bias[h][min(p - j, last)] to the scaled
-//                     score; o may be multiplied by one number (post).  Query head h reads key head h / (QH / KH)
+//                     score; o may be multiplied by one number (post) and by sigmoid(hgate[token, head]).  Query head h reads key head h / (QH / KH)
 //                     and value head h / (QH / VH); the value may be the first V numbers of the key row.
 //   head_norm_gate    per (token, head): u / sqrt(mean(u^2) + eps) * w * post * act(gate), with u one
 //                     head's row or the difference first - coef * second of two attention maps
@@ -35,8 +36,8 @@ __device__ __forceinline__ int clamp_pos(int pos, int rows) { return pos < 0 ? 0
 // nw [D] fp32 or null: the head is first set to unit RMS (eps inside the root) times that weight.
 template <typename IN, typename OUT>
 __device__ __forceinline__ void turn_head(OUT* dst, const IN* src, int D, const float* cs, int pairs, int halves, int lane,
-                                          const float* nw = nullptr, float eps = 0.f) {
-  float k = 1.f;
+                                          const float* nw = nullptr, float eps = 0.f, float post = 1.f) {
+  float k = post;
   if (nw) {
     float ss = 0.f;
     for (int i = lane; i < D; i += 64) {
@@ -44,14 +45,15 @@ __device__ __forceinline__ void turn_head(OUT* dst, const IN* src, int D, const 
       ss += x * x;
     }
     ss = pk::wave_sum(ss);
-    k = 1.f / sqrtf(ss / static_cast<float>(D) + eps);
+    k = post / sqrtf(ss / static_cast<float>(D) + eps);
   }
+  const bool scaled = nw != nullptr || post != 1.f;
   for (int i = lane; i < pairs; i += 64) {
     const int iu = halves ? i : 2 * i, iv = halves ? i + pairs : 2 * i + 1;
     float u = ld<IN>(src + iu), v = ld<IN>(src + iv);
-    if (nw) {
-      u = u * k * nw[iu];
-      v = v * k * nw[iv];
+    if (scaled) {
+      u = u * k * (nw ? nw[iu] : 1.f);
+      v = v * k * (nw ? nw[iv] : 1.f);
     }
     const float c = cs[2 * i], s = cs[2 * i + 1];
     st<OUT>(dst + iu, u * c - v * s);
@@ -59,7 +61,7 @@ __device__ __forceinline__ void turn_head(OUT* dst, const IN* src, int D, const 
   }
   for (int i = 2 * pairs + lane; i < D; i += 64) {
     const float x = ld<IN>(src + i);
-    st<OUT>(dst + i, nw ? x * k * nw[i] : x);
+    st<OUT>(dst + i, scaled ? x * k * (nw ? nw[i] : 1.f) : x);
   }
 }
 
@@ -68,15 +70,17 @@ __global__ void __launch_bounds__(64)
 rotate_cache_kernel(T* __restrict__ q_out, const T* __restrict__ proj, int64_t stride, const int* __restrict__ positions,
                     const int* __restrict__ slot_mapping, const float* __restrict__ table, int pairs, int table_rows,
                     int halves, T* __restrict__ k_cache, T* __restrict__ v_cache, int QH, int KH, int VH, int D, int V,
-                    int bs, const float* __restrict__ q_norm, const float* __restrict__ k_norm, int v_unit, float eps) {
+                    int bs, const float* __restrict__ q_norm, const float* __restrict__ k_norm, int v_unit, float eps,
+                    float temp_coef, int temp_every) {
   const int t = blockIdx.x, item = blockIdx.y, lane = threadIdx.x;
   const int slot = slot_mapping[t];
   const T* row = proj + static_cast<int64_t>(t) * stride;
   const float* cs = table ? table + static_cast<int64_t>(clamp_pos(positions[t], table_rows)) * pairs * 2 : nullptr;
   const int np = cs ? pairs : 0;
   if (item < QH) {
+    const float post = temp_every > 0 ? 1.f + temp_coef * logf(static_cast<float>((max(positions[t], 0) + 1) / temp_every + 1)) : 1.f;
     turn_head<T, T>(q_out + (static_cast<int64_t>(t) * QH + item) * D, row + static_cast<int64_t>(item) * D, D, cs, np,
-                    halves, lane, q_norm, eps);
+                    halves, lane, q_norm, eps, post);
   } else if (item < QH + KH) {
     if (slot < 0) return;
     const int g = item - QH;
@@ -171,6 +175,8 @@ struct MaskedArgs {
   const float* bias;  // [QH, bias_n] added to the scaled scores by distance (the last entry for all beyond) or null
   int bias_n;
   float post;
+  const void* hgate;  // [T, QH] pre-sigmoid factors of a head's result, cache element type, or null
+  int64_t hgate_stride;
   // decoded tokens on the matrix cores: the band's keys cut into n_parts runs of `part` keys,
   // partial sums in the workspace (merged by masked_merge_kernel)
   int part, n_parts;
@@ -183,6 +189,11 @@ __device__ __forceinline__ int first_key(int pos, int window, int chunk) {
   if (window > 0) lo = max(lo, pos - window + 1);
   if (chunk > 0) lo = max(lo, pos / chunk * chunk);
   return lo;
+}
+
+template <typename T>
+__device__ __forceinline__ float head_factor(const void* gate, int64_t stride, int64_t tok, int h) {
+  return gate ? sigmoidf(ld<T>(static_cast<const T*>(gate) + tok * stride + h)) : 1.f;
 }
 
 // The keys a tile of rows walks: kept tiles [0, kept) in front of the band's first tile, then the band.
@@ -328,8 +339,8 @@ __global__ void __launch_bounds__(kThreads) masked_attention_kernel(MaskedArgs a
     __syncthreads();
   }
   const float l = l_s[qi];
-  const float inv = l > 0.f ? a.post / l : 0.f;
   if (!live) return;
+  const float inv = l > 0.f ? a.post / l * head_factor<T>(a.hgate, a.hgate_stride, q0 + my_tl, my_h) : 0.f;
   const int64_t at = static_cast<int64_t>(q0 + my_tl) * a.out_ts + static_cast<int64_t>(my_h) * a.out_hs;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
@@ -618,7 +629,7 @@ __global__ void __launch_bounds__(64 * NW, (D <= 128 && V <= 128) ? 4 : 1) maske
     return;
   }
   if (valid) {
-    const float inv = l_run > 0.f ? a.post / l_run : 0.f;
+    const float inv = l_run > 0.f ? a.post / l_run * head_factor<bf16_t>(a.hgate, a.hgate_stride, q0 + tl, h) : 0.f;
     const int64_t at = static_cast<int64_t>(q0 + tl) * a.out_ts + static_cast<int64_t>(h) * a.out_hs + 4 * g;
 #pragma unroll
     for (int rt = 0; rt < NRT; ++rt) {
@@ -641,7 +652,7 @@ template <typename T>
 __global__ void __launch_bounds__(128)
 masked_merge_kernel(void* __restrict__ out, int64_t out_ts, int64_t out_hs, int out_f32, const float* __restrict__ ws_o,
                     const float* __restrict__ ws_ml, const int* __restrict__ cu_q, const float* __restrict__ sink,
-                    int n_parts, int QH, int V, float post) {
+                    int n_parts, int QH, int V, float post, const void* __restrict__ hgate, int64_t hgate_stride) {
   __shared__ float wgt[64];
   const int s = blockIdx.x, h = blockIdx.y;
   const int tok = cu_q[s];
@@ -655,7 +666,7 @@ masked_merge_kernel(void* __restrict__ out, int64_t out_ts, int64_t out_hs, int 
     const float w = m == -INFINITY ? 0.f : exp2f(m - M);
     float L = pk::wave_sum(w * l);
     if (sink) L += exp2f(sk - M);
-    wgt[p] = L > 0.f ? w * post / L : 0.f;
+    wgt[p] = L > 0.f ? w * post / L * head_factor<T>(hgate, hgate_stride, tok, h) : 0.f;
   }
   __syncthreads();
   const int64_t at = static_cast<int64_t>(tok) * out_ts + static_cast<int64_t>(h) * out_hs;
@@ -758,19 +769,21 @@ head_norm_gate_kernel(OT* __restrict__ out, int64_t out_stride, const float* __r
 }  // namespace
 
 // proj [T, QH*D | KH*D | VH*V] rows `stride` elements apart; table [table_rows, pairs, 2] fp32 or null;
-// q_norm / k_norm [D] fp32 or null: unit RMS times the weight before the rotation; v_unit: v set to unit RMS
+// q_norm / k_norm [D] fp32 or null: unit RMS times the weight before the rotation; v_unit: v set to unit RMS;
+// temp_every > 0: q times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
 PK_EXPORT int pkm_rotate_cache(void* q_out, const void* proj, long long stride, const void* positions,
                                const void* slot_mapping, const void* table, int pairs, int table_rows, int halves,
                                void* k_cache, void* v_cache, int T, int QH, int KH, int VH, int D, int V, int bs,
-                               const void* q_norm, const void* k_norm, int v_unit, float eps, int dt, hipStream_t stream) {
+                               const void* q_norm, const void* k_norm, int v_unit, float eps, float temp_coef,
+                               int temp_every, int dt, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (D < 1 || V < 1 || 2 * pairs > D || (table && table_rows < 1) || bs < 1) return -1;
+  if (D < 1 || V < 1 || 2 * pairs > D || (table && table_rows < 1) || bs < 1 || temp_every < 0) return -1;
   const dim3 grid(T, QH + KH + VH);
   PKM_DISPATCH(dt, E, rotate_cache_kernel<E><<<grid, 64, 0, stream>>>(
                           static_cast<E*>(q_out), static_cast<const E*>(proj), stride, static_cast<const int*>(positions),
                           static_cast<const int*>(slot_mapping), static_cast<const float*>(table), pairs, table_rows,
                           halves, static_cast<E*>(k_cache), static_cast<E*>(v_cache), QH, KH, VH, D, V, bs,
-                          static_cast<const float*>(q_norm), static_cast<const float*>(k_norm), v_unit, eps));
+                          static_cast<const float*>(q_norm), static_cast<const float*>(k_norm), v_unit, eps, temp_coef, temp_every));
   return PK_CHECK_LAUNCH();
 }
 
@@ -806,13 +819,13 @@ PK_EXPORT int pkm_latent_query(void* out, const void* q_lat, const void* q, cons
 
 // v_cache == k_cache: the value of a key is the first V numbers of its key row.  keep: keys below it stay visible;
 // bias [QH, bias_n] fp32 or null; post multiplies the result; fine: softmax weights to 16 bits on the matrix cores
-// (always with keep or bias)
+// (always with keep or bias); hgate [T, QH] rows hgate_stride elements apart (type dt) or null
 PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs, int out_dt, const void* q, int q_dt,
                                    const void* k_cache, const void* v_cache, int v_width, const void* block_tables,
                                    long long bt_stride, const void* cu_q, const void* context_lens, const void* sink,
                                    int n_seqs, int T, int QH, int KH, int VH, int D, int V, int bs, float scale, int window,
-                                   int chunk, int keep, const void* bias, int bias_n, float post, int fine, int num_decode,
-                                   void* ws_o, void* ws_ml, int part, int n_parts, int dt, hipStream_t stream) {
+                                   int chunk, int keep, const void* bias, int bias_n, float post, int fine, const void* hgate,
+                                   long long hgate_stride, int num_decode, void* ws_o, void* ws_ml, int part, int n_parts, int dt, hipStream_t stream) {
   if (n_seqs <= 0 || T <= 0) return 0;
   if (KH < 1 || VH < 1 || QH % KH || KH % VH || V < 1 || V > 512 || V > v_width || D < 1) return -1;
   if ((q_dt != dt && q_dt != kF32) || (out_dt != dt && out_dt != kF32)) return -1;
@@ -824,7 +837,8 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
   MaskedArgs a{out, out_ts, out_hs, out_dt == kF32, q, q_dt == kF32, k_cache, v_cache, v_width,
                static_cast<const int*>(block_tables), bt_stride, static_cast<const int*>(cu_q),
                static_cast<const int*>(context_lens), static_cast<const float*>(sink), n_seqs, QH, KH, VH, D, V, bs, bk,
-               scale, window, chunk, keep, static_cast<const float*>(bias), bias_n, post, 0, 1, nullptr, nullptr};
+               scale, window, chunk, keep, static_cast<const float*>(bias), bias_n, post, hgate, hgate_stride, 0, 1,
+               nullptr, nullptr};
   const bool finer = fine || keep > 0 || bias;
   const int R = QH / KH;
   if (g_masked_mfma && dt == kBF16 && q_dt == kBF16 && bs % 32 == 0 && v_width % 8 == 0 && out_ts % 4 == 0 && out_hs % 4 == 0 &&
@@ -843,7 +857,7 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
       int rc = finer ? launch_mfma<true, true>(d, nd, alias, stream) : launch_mfma<true, false>(d, nd, alias, stream);
       if (rc) return rc;
       masked_merge_kernel<bf16_t><<<dim3(nd, QH), 128, 0, stream>>>(out, out_ts, out_hs, a.out_f32, d.ws_o, d.ws_ml, d.cu_q,
-                                                                    d.sink, n_parts, QH, V, post);
+                                                                    d.sink, n_parts, QH, V, post, hgate, hgate_stride);
       rc = PK_CHECK_LAUNCH();
       if (rc) return rc;
     }
@@ -851,7 +865,7 @@ PK_EXPORT int pkm_masked_attention(void* out, long long out_ts, long long out_hs
       MaskedArgs p = a;
       p.n_seqs = n_seqs - nd;
       p.block_tables += static_cast<int64_t>(nd) * bt_stride;
-      p.cu_q += nd;
+      p.cu_q += nd;  // holds token numbers of the whole step, so q, out and hgate keep their bases
       p.context_lens += nd;
       return finer ? launch_mfma<false, true>(p, T - nd, alias, stream) : launch_mfma<false, false>(p, T - nd, alias, stream);
     }

@@ -1,5 +1,6 @@
-"""Model families: Llama-3 (8B / 70B), Mixtral-8x7B (TP/EP-aware), Sapapel, Kivezen, Nopunex, Bibezen and Lefuvik (single GPU)."""
-from .config import PRESETS, BibezenConfig, KivezenConfig, LefuvikConfig, ModelConfig, NopunexConfig, SapapelConfig, get_config
+"""Model families: Llama-3 (8B / 70B), Mixtral-8x7B (TP/EP-aware), Sapapel, Kivezen, Nopunex, Bibezen, Lefuvik and Vagelix (single GPU)."""
+from .config import (PRESETS, BibezenConfig, KivezenConfig, LefuvikConfig, ModelConfig, NopunexConfig, SapapelConfig, VagelixConfig,
+                     get_config)
 from .llama import LlamaForCausalLM
 
 
@@ -19,6 +20,9 @@ def build_model(cfg, st, dtype, device):
     if isinstance(cfg, LefuvikConfig):
         from .lefuvik import LefuvikForCausalLM
         return LefuvikForCausalLM(cfg, st, dtype, device)
+    if isinstance(cfg, VagelixConfig):
+        from .vagelix import VagelixForCausalLM
+        return VagelixForCausalLM(cfg, st, dtype, device)
     if cfg.is_moe:
         from .mixtral import MixtralForCausalLM
         return MixtralForCausalLM(cfg, st, dtype, device)
@@ -26,4 +30,4 @@ def build_model(cfg, st, dtype, device):
 
 
 __all__ = ["PRESETS", "ModelConfig", "SapapelConfig", "KivezenConfig", "NopunexConfig", "BibezenConfig", "LefuvikConfig",
-           "get_config", "LlamaForCausalLM", "build_model"]
+           "VagelixConfig", "get_config", "LlamaForCausalLM", "build_model"]

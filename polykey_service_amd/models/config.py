@@ -122,6 +122,7 @@ class LayerSpec:
     type: str
     mixer: object    # the mixer's spec (LatentAttentionSpec, SinkAttentionSpec, LightningSpec)
     mlp: object      # the feed-forward's spec, None: no feed-forward
+    weights_of: int = -1    # >= 0: the layer whose weights this one uses (with a cache / state of its own)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -363,7 +364,10 @@ class DiffAttentionSpec:
     """Grouped-query differential attention: two softmax maps per head over the same values, the
     second subtracted with one learned factor (offset ``diff``), the difference set to unit RMS per
     head and scaled by 1 - ``diff``, then gated by a sigmoid of the mixer's input.  ``chunk`` > 0:
-    a key is visible only inside the query's block of ``chunk`` positions (counted from 0)."""
+    a key is visible only inside the query's block of ``chunk`` positions (counted from 0).  Optional:
+    ``qk_norm`` weighted unit-RMS query / key heads (one weight for all heads and maps); ``temp`` =
+    (coef, every): the query at position p times 1 + coef ln(floor((p + 1) / every) + 1); no ``gate``;
+    ``fine``: softmax weights kept to 16 bits on the matrix cores."""
     heads: int
     kv_heads: int
     dim: int
@@ -372,18 +376,26 @@ class DiffAttentionSpec:
     diff: float
     rot: Optional[RotarySpec] = None
     chunk: int = 0
+    qk_norm: bool = False
+    temp: Optional[tuple] = None
+    gate: bool = True
+    fine: bool = False
 
 
 @dataclasses.dataclass(frozen=True)
 class DeltaSpec:
     """Gated delta rule: per head a [dim, vdim] fp32 memory that decays by a data-dependent gate,
     is corrected along the new unit key towards the new value, and is read with the unit query;
-    q, k, v pass a causal per-channel filter of ``conv`` taps and SiLU first."""
+    q, k, v pass a causal per-channel filter of ``conv`` taps and SiLU first.  The gate is one number
+    per head, or (``decay_rank`` > 0) one per head and key channel from a low-rank projection;
+    ``gate_rank`` > 0: the output gate comes from a low-rank projection too."""
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     conv: int
+    decay_rank: int = 0
+    gate_rank: int = 0
 
 
 @dataclasses.dataclass(frozen=True)
@@ -956,10 +968,198 @@ class LefuvikConfig:
                    logit_softcap=30.0)
 
 
+@dataclasses.dataclass(frozen=True)
+class ChunkAttentionSpec:
+    """Grouped-query softmax attention inside blocks of ``chunk`` positions counted from position 0 (0:
+    every earlier key): biased query / key projections, the projected keys as values, one weighted RMS
+    norm over all query (key) heads together, a partial rotation, ``sink`` extra exp(0) terms in the
+    softmax denominator and one sigmoid gate per head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    rot: Optional[RotarySpec] = None
+    chunk: int = 0
+    sink: float = 1.0
+
+    @property
+    def vdim(self) -> int:
+        return self.dim
+
+
+@dataclasses.dataclass(frozen=True)
+class StepScanSpec:
+    """State-space duality: per head a [state, vdim] fp32 memory whose decay and input scale come from one
+    step size per head, input / output vectors shared by ``groups`` of heads, a causal filter of ``conv``
+    taps and SiLU in front, a SiLU gate and an RMS norm in ``norm_groups`` equal parts behind."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclasses.dataclass(frozen=True)
+class VagelixConfig:
+    """Vagelix: a normed embedding starts one fp32 residual stream; sublayers read the stream itself and
+    only their outputs are normed.  Mixers are ``parallel`` (chunked attention beside the gated delta
+    rule with per-channel decays, both outputs normed and averaged), ``mamba2`` (state-space duality)
+    or ``attention`` (causal differential attention with a query temperature); SiLU-gated dense
+    feed-forwards, or none.  A layer may use another one's weights with a cache / state of its own.
+    Logits reuse the embedding table.  Read from a checkpoint folder's config.json ("architecture":
+    "Vagelix")."""
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: tuple
+    rms_eps: float
+    max_position: int = 1 << 20     # the rotation tables are built for the engine's max_model_len
+    bos_token_id: int = 0
+    eos_token_id: int = -1
+    init_std: float = 0.05
+    family: str = "vagelix"
+    is_moe: bool = False
+    experts_per_token: int = 0
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def runs(self) -> tuple:
+        return tuple(range(len(self.layers)))
+
+    @property
+    def needs_state(self) -> bool:
+        return any(l.type != "attention" for l in self.layers)
+
+    def num_params(self) -> int:
+        W = self.hidden_size
+        n = self.vocab_size * W + 2 * W
+        for l in self.layers:
+            if l.weights_of >= 0:
+                continue
+            m, f = l.mixer, l.mlp
+            n += W * (2 if f is not None else 1) + (3 * W * f.ff if f is not None else 0)
+            if l.type == "parallel":
+                a, b = m.left, m.right
+                qk, c = (a.heads + a.kv_heads) * a.dim, 2 * b.kv_heads * b.dim + b.heads * b.vdim
+                n += qk * (W + 2) + a.heads * W * (1 + a.dim) + 2 * W
+                n += c * (W + b.conv) + b.heads * (W + 1) + b.vdim + b.heads * b.vdim * W
+                n += b.decay_rank * (W + b.heads * b.dim) + b.heads * b.dim + b.gate_rank * (W + b.heads * b.vdim)
+            elif l.type == "mamba2":
+                c = m.inner + 2 * m.groups * m.state
+                n += W * (m.inner + c + m.heads) + c * (m.conv + 1) + 3 * m.heads + m.inner * (1 + W)
+            else:
+                n += W * (2 * (m.heads + m.kv_heads) * m.dim + (m.kv_heads + m.heads) * m.vdim) + 6 * m.dim
+        return n
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        n = 0
+        for l in self.layers:
+            if l.type == "parallel":
+                n += l.mixer.left.kv_heads * 2 * l.mixer.left.dim
+            elif l.type == "attention":
+                n += l.mixer.kv_heads * (2 * l.mixer.dim + l.mixer.vdim)
+        return n * dtype_bytes
+
+    @classmethod
+    def _mixer(cls, kind: str, m: dict):
+        if kind == "parallel":
+            a, b = m["left"], m["right"]
+            r = a.get("rot")
+            rot = RotarySpec(int(r["dims"]), float(r["base"]), None, halves=True) if r and int(r["dims"]) else None
+            left = ChunkAttentionSpec(int(a["heads"]), int(a.get("kv_heads", a["heads"])), int(a["dim"]), float(a["scale"]), rot,
+                                      int((a.get("mask") or {}).get("size") or 0))
+            right = DeltaSpec(int(b["heads"]), int(b.get("kv_heads", b["heads"])), int(b["dim"]), int(b.get("vdim", b["dim"])),
+                              int(b["conv"]))
+            if int(a.get("vdim", a["dim"])) != left.dim:
+                raise ValueError("Vagelix: the keys are the values, so vdim must equal dim")
+            if left.heads % left.kv_heads or right.heads % right.kv_heads or right.conv < 1:
+                raise ValueError("Vagelix: heads must be a multiple of kv_heads and conv at least 1")
+            if rot is not None and (rot.dims % 2 or rot.dims > left.dim):
+                raise ValueError("Vagelix: rot.dims must be even and at most dim")
+            return ParallelSpec(left, right, 0.5, 0.5)
+        if kind == "mamba2":
+            s = StepScanSpec(int(m["heads"]), int(m["vdim"]), int(m["state"]), int(m.get("groups", 1)), int(m["conv"]),
+                             int(m.get("norm_groups", 1)))
+            if s.heads % s.groups or s.inner % s.norm_groups or s.conv < 1:
+                raise ValueError("Vagelix: heads must divide by groups, heads * vdim by norm_groups, conv be at least 1")
+            return s
+        if kind == "attention":
+            t = m.get("q_temp")
+            if t is not None and (int(t["every"]) != t["every"] or int(t["every"]) < 1):
+                raise ValueError("Vagelix: q_temp.every must be a positive whole number")
+            s = DiffAttentionSpec(int(m["heads"]), int(m.get("kv_heads", m["heads"])), int(m["dim"]), int(m.get("vdim", m["dim"])),
+                                  float(m["scale"]), float(m["diff"]), None, 0, True,
+                                  (float(t["coef"]), int(t["every"])) if t is not None else None, False, True)
+            if s.heads % s.kv_heads:
+                raise ValueError("Vagelix: attention heads must be a multiple of kv_heads")
+            return s
+        raise ValueError(f"Vagelix: unknown mixer type {kind!r}")
+
+    @classmethod
+    def from_json(cls, c: dict, name: str = "vagelix") -> "VagelixConfig":
+        layers = []
+        for l in c["layers"]:
+            f, src = l.get("mlp"), l.get("weights_of")
+            if f is not None and f.get("kind") != "dense":
+                raise ValueError(f"Vagelix: unknown feed-forward kind {f.get('kind')!r}")
+            layers.append(LayerSpec(l["type"], cls._mixer(l["type"], l["mixer"]), GatedFFSpec(int(f["ff"])) if f is not None else None,
+                                    -1 if src is None else int(src)))
+        return cls(name=name, vocab_size=int(c["vocab"]), hidden_size=int(c["width"]), layers=cls._resolve(layers),
+                   rms_eps=float(c["norm"]["eps"]))
+
+    @staticmethod
+    def _resolve(layers: list) -> tuple:
+        """Every ``weights_of`` names a layer with weights of its own and the same sizes."""
+        out = []
+        for i, l in enumerate(layers):
+            j, seen = i, {i}
+            while layers[j].weights_of >= 0:
+                j = layers[j].weights_of
+                if j >= len(layers) or j in seen:
+                    raise ValueError(f"Vagelix: layer {i} has no layer to take its weights from")
+                seen.add(j)
+            o = layers[j]
+            if (o.type, o.mixer, o.mlp) != (l.type, l.mixer, l.mlp):
+                raise ValueError(f"Vagelix: layer {i} differs from layer {j}, whose weights it uses")
+            out.append(dataclasses.replace(l, weights_of=j if j != i else -1))
+        return tuple(out)
+
+    @classmethod
+    def uniform(cls, name: str, vocab: int, width: int, pattern: str, heads: int, kv_heads: int, dim: int, ff: int,
+                chunk: int = 1024, state: int = 128, scan_dim: int = 64, groups: int = 1, rank: int = 128,
+                every: int = 1024) -> "VagelixConfig":
+        """``pattern``: one letter per layer, P parallel / S state-space / A attention (lower case: without
+        a feed-forward); a digit uses the weights of that layer."""
+        layers = []
+        for ch in pattern:
+            if ch.isdigit():
+                layers.append(dataclasses.replace(layers[int(ch)], weights_of=int(ch)))
+                continue
+            up = ch.upper()
+            if up == "P":
+                mixer = ParallelSpec(ChunkAttentionSpec(heads, kv_heads, dim, dim ** -0.5, RotarySpec(dim // 2, 1e4, None, True), chunk),
+                                     DeltaSpec(heads, kv_heads, dim, dim, 4, rank, rank), 0.5, 0.5)
+            elif up == "S":
+                mixer = StepScanSpec(2 * width // scan_dim, scan_dim, state, groups, 4, groups)
+            else:
+                mixer = DiffAttentionSpec(heads, kv_heads, dim, dim, dim ** -0.5, 0.3, None, 0, True, (0.1, every), False, True)
+            layers.append(LayerSpec({"P": "parallel", "S": "mamba2", "A": "attention"}[up], mixer,
+                                    GatedFFSpec(ff) if ch.isupper() else None))
+        return cls(name=name, vocab_size=vocab, hidden_size=width, layers=cls._resolve(layers), rms_eps=1e-5)
+
+
 # config.json "architecture" -> reader (checkpoints that are not HF Llama / Mixtral folders)
 ARCHITECTURES = {"Sapapel": SapapelConfig.from_json, "Kivezen": KivezenConfig.from_json,
                  "Nopunex": NopunexConfig.from_json, "Bibezen": BibezenConfig.from_json,
-                 "Lefuvik": LefuvikConfig.from_json}
+                 "Lefuvik": LefuvikConfig.from_json, "Vagelix": VagelixConfig.from_json}
 
 PRESETS["tiny-sapapel"] = SapapelConfig.uniform("tiny-sapapel", 512, 128, 3, 4, 16, 32, 48, 64, 6, 2)
 # speed measurements (random weights): layer shapes of small production MoE models, and the
@@ -1005,6 +1205,15 @@ PRESETS["tiny-lefuvik"] = LefuvikConfig.uniform("tiny-lefuvik", 512, 128, "pRMSP
 # ungated experts half as wide again as the gated ones (equal weights per expert)
 PRESETS["lefuvik-2k"] = LefuvikConfig.uniform("lefuvik-2k", 32000, 2048, "RPMPRPSP", 16, 4, 128, 6144)
 PRESETS["lefuvik-4k"] = LefuvikConfig.uniform("lefuvik-4k", 32000, 4096, "RPMP", 32, 8, 128, 12288, 8, 2, 3072, rec_blocks=32)
+
+
+PRESETS["tiny-vagelix"] = VagelixConfig.uniform("tiny-vagelix", 512, 128, "PSa0A", 4, 2, 32, 256, chunk=24, state=16, scan_dim=32,
+                                                groups=2, rank=16, every=16)
+# speed measurements beside nopunex-2k / nopunex-4k (the closest family: differential attention, chunks, the
+# gated delta rule, dense feed-forwards on one fp32 stream): the same width, depth, heads, KV heads, head and
+# feed-forward size
+PRESETS["vagelix-2k"] = VagelixConfig.uniform("vagelix-2k", 32000, 2048, "PSAPSA03", 16, 4, 128, 4608)
+PRESETS["vagelix-4k"] = VagelixConfig.uniform("vagelix-4k", 32000, 4096, "PSAP", 32, 8, 128, 6144)
 
 
 def get_config(name_or_path: str):

@@ -63,24 +63,29 @@ class DiffAttention(nn.Module):
     def __init__(self, spec, width: int):
         super().__init__()
         self.spec, self.width = spec, width
-        self.w_in = None   # [2H*D | 2G*D | G*V | H*V, W]: q (regrouped) | k | v | gate rows
+        self.w_in = None   # [2H*D | 2G*D | G*V | H*V, W]: q (regrouped) | k | v | gate rows (gate: only with one)
         self.w_o = None    # [W, H*V]
         self.lam = 0.0     # exp(lq1 . lk1) - exp(lq2 . lk2) + diff
         self.table = None  # [positions, pairs, 2] fp32 (cos, sin); None: no rotation
+        self.q_norm = self.k_norm = None    # [D] fp32 (qk_norm)
         self.w_in_p = self.w_o_p = None
 
     def pack(self) -> None:
         self.w_in_p, self.w_o_p = _packed(self.w_in), _packed(self.w_o)
 
-    def set(self, q, k, v, g, o, lq1, lk1, lq2, lk2, dtype, device) -> None:
+    def set(self, q, k, v, g, o, lq1, lk1, lq2, lk2, dtype, device, q_norm=None, k_norm=None) -> None:
         s = self.spec
         H, G, D, V, W = s.heads, s.kv_heads, s.dim, s.vdim, self.width
         assert q.shape == (2 * H * D, W) and k.shape == (2 * G * D, W) and v.shape == (G * V, W)
-        assert g.shape == (H * V, W) and o.shape == (W, H * V)
+        assert (g is not None) == s.gate and (g is None or g.shape == (H * V, W)) and o.shape == (W, H * V)
+        assert (q_norm is not None) == (k_norm is not None) == s.qk_norm
+        if s.qk_norm:
+            assert q_norm.numel() == D == k_norm.numel()
+            self.q_norm, self.k_norm = (_p(t.to(device=device, dtype=torch.float32).reshape(-1)) for t in (q_norm, k_norm))
         assert s.rot is None or (s.rot.dims % 2 == 0 and s.rot.dims <= D)
         r = H // G
         q = q.reshape(G, r, 2, D, W).permute(0, 2, 1, 3, 4).reshape(2 * H * D, W)
-        self.w_in = _p(_pad_rows(torch.cat([q, k, v, g], 0)).to(device=device, dtype=dtype))
+        self.w_in = _p(_pad_rows(torch.cat([q, k, v] + ([g] if s.gate else []), 0)).to(device=device, dtype=dtype))
         self.w_o = _p(o.to(device=device, dtype=dtype))
         dot = lambda a, b: float((a.double().reshape(-1) * b.double().reshape(-1)).sum())
         self.lam = math.exp(dot(lq1, lk1)) - math.exp(dot(lq2, lk2)) + s.diff
@@ -91,11 +96,12 @@ class DiffAttention(nn.Module):
         n = 2 * (H + G) * D + G * V
         proj = _project(h, self.w_in, self.w_in_p)
         q = ma_ops.rotate_cache(proj[:, :n], positions, md.slot_mapping, self.table, True, cache[0], cache[1],
-                                2 * H, 2 * G, G, D, V)
+                                2 * H, 2 * G, G, D, V, q_norm=self.q_norm, k_norm=self.k_norm, eps=eps, temp=s.temp)
         a = ma_ops.masked_attention(q, cache[0], cache[1], V, md.block_tables, md.cu_q, md.context_lens, md.num_seqs,
-                                    s.scale, chunk=s.chunk, num_decode=md.num_decode)
-        o = ma_ops.head_norm_gate(a, H, V, eps, proj[:, n:n + H * V], ma_ops.GATE_SIGMOID, h.dtype, post=1.0 - s.diff,
-                                  pair_group=H // G, coef=self.lam)
+                                    s.scale, chunk=s.chunk, fine=s.fine, num_decode=md.num_decode)
+        o = ma_ops.head_norm_gate(a, H, V, eps, proj[:, n:n + H * V] if s.gate else None,
+                                  ma_ops.GATE_SIGMOID if s.gate else ma_ops.GATE_NONE, h.dtype,
+                                  post=1.0 - s.diff, pair_group=H // G, coef=self.lam)
         return _project(o, self.w_o, self.w_o_p, partial=True)
 
 

@@ -94,6 +94,38 @@ def hyper_step(xs: torch.Tensor, y, close: Optional[tuple], open_: Optional[tupl
     return act, z32
 
 
+def pair_step(x: torch.Tensor, ya, yb, wa: torch.Tensor, wb: torch.Tensor, ca: float, cb: float, post_w: torch.Tensor, eps: float,
+              act_dtype: torch.dtype) -> torch.Tensor:
+    """Closes a sublayer of two branches on one stream x fp32 [T, 1, W] in place:
+
+        y = ca U(ya) wa + cb U(yb) wb        x <- x + U(y) post_w        U(u) = u / sqrt(mean(u^2) + eps)
+
+    ``ya``, ``yb``: [T, W] tensors of one element type, or the decode GEMM's unreduced split-K slabs.  Returns
+    x in ``act_dtype`` (the next sublayer's input)."""
+    T, S, W = x.shape
+    assert S == 1 and x.dtype == torch.float32 and x.is_contiguous()
+    act = torch.empty((T, W), dtype=act_dtype, device=x.device)
+    if not x.is_cuda:
+        unit = lambda u, w: u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * w
+        x[:, 0] += unit(ca * unit(ya.float(), wa) + cb * unit(yb.float(), wb), post_w)
+        act.copy_(x[:, 0])
+        return act
+
+    def rows(y):
+        if isinstance(y, gemm.Partial):
+            assert y.M == T and y.N == W
+            return y.view()[0], y.S
+        assert y.shape == (T, W) and y.is_contiguous()
+        return y, 1
+    (ya, na), (yb, nb) = rows(ya), rows(yb)
+    for w in (wa, wb, post_w):
+        assert w.dtype == torch.float32 and w.numel() == W
+    native.call("pkm_pair_step", x.data_ptr(), T, W, ya.data_ptr(), na, native.dt_code(ya.dtype), yb.data_ptr(), nb,
+                native.dt_code(yb.dtype), wa.data_ptr(), wb.data_ptr(), float(ca), float(cb), post_w.data_ptr(), float(eps),
+                act.data_ptr(), native.dt_code(act_dtype), native.stream_ptr())
+    return act
+
+
 def spread_rows(table: torch.Tensor, ids: torch.Tensor, S: int, scale: float = 1.0) -> torch.Tensor:
     """xs[t, s] = table[ids[t]] * scale as fp32 for every stream s: [T, S, W]."""
     T, W = ids.numel(), table.shape[1]

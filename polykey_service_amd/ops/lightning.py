@@ -1,5 +1,5 @@
-"""Lightning attention: linear attention with one constant decay per head and an fp32 state per
-(sequence, head) carried from step to step (csrc/mixers/lightning.hip; PyTorch on CPU).
+"""Lightning attention: linear attention with one constant decay per head (or one per step and head) and an
+fp32 state per (sequence, head) carried from step to step (csrc/mixers/lightning.hip; PyTorch on CPU).
 
     S_t = decay_h * S_{t-1} + k_t v_t^T        o_t = S_t^T q_t        q, k, v = silu(projections)
 
@@ -82,6 +82,64 @@ def retention(qkv: torch.Tensor, state: torch.Tensor, decay: torch.Tensor, table
                 native.ptr(table), table.shape[1] if table is not None else 0, table.shape[0] if table is not None else 0,
                 float(k_scale), cu_q.data_ptr(), positions.data_ptr(), slots.data_ptr(), n_seqs, T, H, D, V,
                 native.dt_code(qkv.dtype), native.stream_ptr())
+    return out
+
+
+def step_scan(xbc: torch.Tensor, dt: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor,
+              state: torch.Tensor, cu_q: torch.Tensor, n_seqs: int, positions: torch.Tensor, slots: torch.Tensor, H: int, N: int,
+              V: int, G: int) -> torch.Tensor:
+    """The recurrence with a step size per (token, head) (state-space duality): d = softplus(dt + dt_bias_h),
+
+        S <- exp(-exp(a_log_h) d) S + d B x^T        y = S^T C + skip_h x        S [N, V] fp32 per head
+
+    xbc [T, H*V x | G*N B | G*N C] (may be a column slice), head h on B / C group h // (H / G); ``dt``
+    [T, H] pre-activations of the same element type (may be a column slice); dt_bias, a_log, skip [H] fp32;
+    ``state`` [slots, H, N, V] fp32.  Returns y [T, H * V] fp32."""
+    T = xbc.shape[0]
+    out = torch.empty((T, H * V), dtype=torch.float32, device=xbc.device)
+    assert xbc.shape[1] == H * V + 2 * G * N and dt.shape == (T, H) and H % G == 0
+    if not xbc.is_cuda:
+        f = xbc.float()
+        x, r = f[:, :H * V].view(T, H, V), H // G
+        b = f[:, H * V:H * V + G * N].view(T, G, N).repeat_interleave(r, 1)
+        c = f[:, H * V + G * N:].view(T, G, N).repeat_interleave(r, 1)
+        d = torch.nn.functional.softplus(dt.float() + dt_bias)
+        dec = torch.exp(-torch.exp(a_log) * d)
+        o3 = out.view(T, H, V)
+        for s in range(n_seqs):
+            a, e, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+            if e <= a:
+                continue
+            S = state[slot].clone() if (slot >= 0 and int(positions[a]) > 0) else torch.zeros((H, N, V))
+            for t in range(a, e):
+                S = dec[t, :, None, None] * S + b[t, :, :, None] * (d[t, :, None] * x[t])[:, None, :]
+                o3[t] = torch.einsum("hnv,hn->hv", S, c[t]) + skip[:, None] * x[t]
+            if slot >= 0:
+                state[slot] = S
+        return out
+    assert xbc.stride(1) == 1 and dt.stride(1) == 1 and dt.dtype == xbc.dtype
+    assert state.is_contiguous() and state.dtype == torch.float32 and state.shape[1:] == (H, N, V)
+    for w in (dt_bias, a_log, skip):
+        assert w.dtype == torch.float32 and w.numel() == H
+    native.call("pkm_step_scan", out.data_ptr(), xbc.data_ptr(), xbc.stride(0), dt.data_ptr(), dt.stride(0), G, dt_bias.data_ptr(),
+                a_log.data_ptr(), skip.data_ptr(), state.data_ptr(), cu_q.data_ptr(), positions.data_ptr(), slots.data_ptr(),
+                n_seqs, T, H, N, V, native.dt_code(xbc.dtype), native.stream_ptr())
+    return out
+
+
+def gated_group_norm(y: torch.Tensor, z: torch.Tensor, w: torch.Tensor, parts: int, eps: float, dtype: torch.dtype) -> torch.Tensor:
+    """u = y * silu(z); each of ``parts`` equal parts of u over its own root mean square, times w [N]: y [T, N]
+    fp32, z [T, N] (may be a column slice) -> [T, N] in ``dtype``."""
+    T, N = y.shape
+    out = torch.empty((T, N), dtype=dtype, device=y.device)
+    assert N % parts == 0 and w.numel() == N and z.shape == (T, N)
+    if not y.is_cuda:
+        u = (y * torch.nn.functional.silu(z.float())).view(T, parts, N // parts)
+        out.copy_((u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps)).view(T, N) * w)
+        return out
+    assert y.dtype == torch.float32 and y.is_contiguous() and w.dtype == torch.float32 and z.stride(1) == 1
+    native.call("pkm_gated_group_norm", out.data_ptr(), y.data_ptr(), z.data_ptr(), z.stride(0), w.data_ptr(), T, N, parts,
+                float(eps), native.dt_code(z.dtype), native.dt_code(dtype), native.stream_ptr())
     return out
 
 

@@ -71,6 +71,11 @@ def distance_bias(rel: torch.Tensor, bias_max: int) -> torch.Tensor:
     return rel.float()[row].t().contiguous()
 
 
+def query_temperature(positions: torch.Tensor, coef: float, every: int) -> torch.Tensor:
+    """1 + coef ln(floor((p + 1) / every) + 1), fp32."""
+    return 1.0 + coef * torch.log(((positions.long() + 1) // every + 1).float())
+
+
 def _write_cache(cache: torch.Tensor, rows: torch.Tensor, slot_mapping: torch.Tensor) -> None:
     """cache [blocks, heads, bs, width] <- rows [T, heads, width] at the tokens' slots (< 0: not)."""
     bs = cache.shape[2]
@@ -82,11 +87,13 @@ def _write_cache(cache: torch.Tensor, rows: torch.Tensor, slot_mapping: torch.Te
 def rotate_cache(proj: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor, table: Optional[torch.Tensor],
                  halves: bool, k_cache: torch.Tensor, v_cache: torch.Tensor, QH: int, KH: int, VH: int, D: int,
                  V: int, q_norm: Optional[torch.Tensor] = None, k_norm: Optional[torch.Tensor] = None,
-                 eps: float = 0.0, v_unit: bool = False) -> torch.Tensor:
+                 eps: float = 0.0, v_unit: bool = False, temp: Optional[tuple] = None) -> torch.Tensor:
     """proj [T, QH*D | KH*D | VH*V] (may be a column slice of a wider projection output): q and k
     heads turn by the token's position (``table`` rows; None: no rotation), k and v go to the paged
     caches.  ``q_norm`` / ``k_norm`` [D] fp32: the heads are first set to unit RMS (``eps`` inside
-    the root) times that weight; ``v_unit``: each value head is set to unit RMS.  Returns q [T, QH, D] in the cache's dtype."""
+    the root) times that weight; ``v_unit``: each value head is set to unit RMS; ``temp`` = (coef, every):
+    the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1).  Returns q [T, QH, D]
+    in the cache's dtype."""
     T = proj.shape[0]
     q = torch.empty((T, QH, D), dtype=k_cache.dtype, device=proj.device)
     if not proj.is_cuda:
@@ -103,6 +110,8 @@ def rotate_cache(proj: torch.Tensor, positions: torch.Tensor, slot_mapping: torc
         if table is not None:
             cs = table[positions.long()]
             qq, kk = turn(qq, cs, halves), turn(kk, cs, halves)
+        if temp is not None:
+            qq = qq * query_temperature(positions, *temp)[:, None, None]
         q.copy_(qq)
         _write_cache(k_cache, kk, slot_mapping)
         _write_cache(v_cache, vv, slot_mapping)
@@ -118,7 +127,45 @@ def rotate_cache(proj: torch.Tensor, positions: torch.Tensor, slot_mapping: torc
                 slot_mapping.data_ptr(), native.ptr(table), table.shape[1] if table is not None else 0,
                 table.shape[0] if table is not None else 0, int(halves), k_cache.data_ptr(), v_cache.data_ptr(), T,
                 QH, KH, VH, D, V, k_cache.shape[2], native.ptr(q_norm), native.ptr(k_norm), int(v_unit), float(eps),
+                float(temp[0]) if temp is not None else 0.0, int(temp[1]) if temp is not None else 0,
                 native.dt_code(k_cache.dtype), native.stream_ptr())
+    return q
+
+
+def row_norm_cache(proj: torch.Tensor, bias: torch.Tensor, q_norm: torch.Tensor, k_norm: torch.Tensor, eps: float,
+                   positions: torch.Tensor, slot_mapping: torch.Tensor, table: Optional[torch.Tensor], halves: bool,
+                   k_cache: torch.Tensor, v_cache: torch.Tensor, QH: int, KH: int, D: int) -> torch.Tensor:
+    """Keys that are their own values, normed over all heads at once: proj [T, QH*D | KH*D] (may be a column
+    slice) plus ``bias`` [(QH + KH) * D] fp32; the value cache takes the key row as it is, then all query
+    (key) heads together are set to unit RMS times ``q_norm`` [QH * D] (``k_norm`` [KH * D]) fp32 and turn by
+    the token's position (``table`` rows; None: no rotation); the key cache takes the turned keys.  Returns
+    q [T, QH, D] in the cache's dtype."""
+    T, n = proj.shape[0], (QH + KH) * D
+    q = torch.empty((T, QH, D), dtype=k_cache.dtype, device=proj.device)
+    assert proj.shape[1] == n == bias.numel() and q_norm.numel() == QH * D and k_norm.numel() == KH * D
+    if not proj.is_cuda:
+        f = proj.float() + bias
+        _write_cache(v_cache, f[:, QH * D:].view(T, KH, D), slot_mapping)
+        unit = lambda u, w: u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * w
+        qq, kk = unit(f[:, :QH * D], q_norm).view(T, QH, D), unit(f[:, QH * D:], k_norm).view(T, KH, D)
+        if table is not None:
+            cs = table[positions.long()]
+            qq, kk = turn(qq, cs, halves), turn(kk, cs, halves)
+        q.copy_(qq)
+        _write_cache(k_cache, kk, slot_mapping)
+        return q
+    assert proj.stride(1) == 1 and proj.dtype == k_cache.dtype == v_cache.dtype
+    assert positions.dtype == torch.int32 and slot_mapping.dtype == torch.int32
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.shape == v_cache.shape
+    assert k_cache.shape[1:] == (KH, k_cache.shape[2], D)
+    assert table is None or (table.dtype == torch.float32 and table.is_contiguous() and 2 * table.shape[1] <= D)
+    for w in (bias, q_norm, k_norm):
+        assert w.dtype == torch.float32 and w.is_contiguous()
+    native.call("pkm_row_norm_cache", q.data_ptr(), proj.data_ptr(), proj.stride(0), bias.data_ptr(), q_norm.data_ptr(),
+                k_norm.data_ptr(), float(eps), positions.data_ptr(), slot_mapping.data_ptr(), native.ptr(table),
+                table.shape[1] if table is not None else 0, table.shape[0] if table is not None else 0, int(halves),
+                k_cache.data_ptr(), v_cache.data_ptr(), T, QH, KH, D, k_cache.shape[2], native.dt_code(k_cache.dtype),
+                native.stream_ptr())
     return q
 
 
@@ -127,7 +174,7 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[t
                      scale: float, window: int = 0, chunk: int = 0, sink: Optional[torch.Tensor] = None,
                      out_dtype: torch.dtype = torch.float32, head_major: bool = False, num_decode: int = 0,
                      keep: int = 0, bias: Optional[torch.Tensor] = None, post: float = 1.0, fine: bool = False,
-                     out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     out: Optional[torch.Tensor] = None, head_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [T, QH, D] (fp32 or the cache's dtype); sequence s owns tokens cu_q[s]:cu_q[s+1], the LAST
     ones of its context_lens[s] cached tokens.  ``v_cache`` None: the value of a key is the first
     ``V`` numbers of its key row (key heads = value heads).  ``sink`` [QH] fp32 logits or None.
@@ -136,7 +183,8 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[t
     in ``out_dtype``.  Scores, softmax and the value sums are fp32.  ``keep``: the first keys that stay
     visible; ``bias`` [QH, n] fp32 (:func:`distance_bias`); ``post`` multiplies the result; ``fine``: the
     matrix-core kernel sees the softmax weights to 16 bits (always with ``keep`` or ``bias``; a single
-    bf16 otherwise); ``out``: write there ([T, QH * V], may be a column slice of a wider row)."""
+    bf16 otherwise); ``out``: write there ([T, QH * V], may be a column slice of a wider row); ``head_gate``
+    [T, QH] in the cache's dtype (may be a column slice): head h's result times its sigmoid."""
     T, QH, D = q.shape
     KH, bs = k_cache.shape[1], k_cache.shape[2]
     vc = k_cache if v_cache is None else v_cache
@@ -176,12 +224,16 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[t
             den = e.sum(-1, keepdim=True)
             if sink is not None:
                 den = den + torch.exp(sink[:, None, None] - m)
-            o3[a:b] = (torch.einsum("htj,jhv->thv", e / den, v) * post).to(out_dtype)
+            o = torch.einsum("htj,jhv->thv", e / den, v) * post
+            if head_gate is not None:
+                o = o * torch.sigmoid(head_gate[a:b].float())[..., None]
+            o3[a:b] = o.to(out_dtype)
         return out
     assert q.is_contiguous() and k_cache.is_contiguous() and vc.is_contiguous() and vc.dtype == k_cache.dtype
     assert block_tables.stride(1) == 1 and (sink is None or (sink.dtype == torch.float32 and sink.numel() == QH))
     assert q.dtype in (torch.float32, k_cache.dtype)
     assert bias is None or (bias.dtype == torch.float32 and bias.is_contiguous() and bias.shape[0] == QH)
+    assert head_gate is None or (head_gate.shape == (T, QH) and head_gate.stride(1) == 1 and head_gate.dtype == k_cache.dtype)
     ts, hs = (V, T * V) if head_major else (out.stride(0), V)
     nd = min(num_decode, n_seqs)
     ws_o = ws_ml = None
@@ -205,7 +257,8 @@ def masked_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[t
                 native.dt_code(q.dtype), k_cache.data_ptr(), vc.data_ptr(), vc.shape[3], block_tables.data_ptr(),
                 block_tables.stride(0), cu_q.data_ptr(), context_lens.data_ptr(), native.ptr(sink), n_seqs, T, QH, KH, VH,
                 D, V, bs, float(scale), int(window), int(chunk), int(keep), native.ptr(bias),
-                bias.shape[1] if bias is not None else 0, float(post), int(fine), nd, native.ptr(ws_o), native.ptr(ws_ml), part, n_parts,
+                bias.shape[1] if bias is not None else 0, float(post), int(fine), native.ptr(head_gate),
+                head_gate.stride(0) if head_gate is not None else 0, nd, native.ptr(ws_o), native.ptr(ws_ml), part, n_parts,
                 native.dt_code(k_cache.dtype), native.stream_ptr())
     return out
 

@@ -106,16 +106,20 @@ MIXER_SIGNATURES = {
     "pkm_join_cast": [P, P, P, I32, I32, I32, P],
     "pkm_silu_mul": [P, P, I32, I32, I32, I32, I32, P],
     "pkm_scale": [P, I64, F32, P],
-    "pkm_rotate_cache": [P, P, I64, P, P, P, I32, I32, I32, P, P, I32, I32, I32, I32, I32, I32, I32, P, P, I32, F32, I32, P],
+    "pkm_rotate_cache": [P, P, I64, P, P, P, I32, I32, I32, P, P, I32, I32, I32, I32, I32, I32, I32, P, P, I32, F32, F32, I32, I32, P],
+    "pkm_row_norm_cache": [P, P, I64, P, P, P, F32, P, P, P, I32, I32, I32, P, P, I32, I32, I32, I32, I32, I32, P],
+    "pkm_gated_group_norm": [P, P, P, I64, P, I32, I32, I32, F32, I32, I32, P],
+    "pkm_step_scan": [P, P, I64, P, I64, I32, P, P, P, P, P, P, P, I32, I32, I32, I32, I32, I32, P],
+    "pkm_pair_step": [P, I32, I32, P, I32, I32, P, I32, I32, P, P, F32, F32, P, F32, P, I32, P],
     "pkm_latent_in": [P, P, P, I64, I32, I32, I32, P, P, F32, P, P, P, I32, I32, I32, I32, I32, I32, P],
     "pkm_latent_query": [P, P, P, P, P, I32, I32, I32, I32, I32, I32, I32, I32, I32, P],
     "pkm_masked_attention": [P, I64, I64, I32, P, I32, P, P, I32, P, I64, P, P, P, I32, I32, I32, I32, I32, I32, I32, I32,
-                             F32, I32, I32, I32, P, I32, F32, I32, I32, P, P, I32, I32, I32, P],
+                             F32, I32, I32, I32, P, I32, F32, I32, P, I64, I32, P, P, I32, I32, I32, P],
     "pkm_masked_decode_part": [I32, I32, I32, I32, I32, I32, I32, I32, I32, I32, I32, I32],
     "pkm_set_masked_mfma": [I32],
     "pkm_head_norm_gate": [P, I64, P, I32, I32, I32, F32, P, I64, I32, I32, P, I32, F32, I32, F32, I32, P],
-    "pkm_conv_unit": [P, P, I64, P, I32, P, P, P, P, P, I32, I32, I32, I32, I32, I32, I32, P],
-    "pkm_delta_rule": [P, P, P, I64, I32, P, P, P, P, P, P, I32, I32, I32, I32, I32, I32, P],
+    "pkm_conv_unit": [P, P, I64, P, I32, P, P, P, P, P, I32, I32, I32, I32, I32, I32, P, P, I64, P, P, I32, I32, P],
+    "pkm_delta_rule": [P, P, P, I64, I32, P, P, P, P, P, P, P, I32, I32, I32, I32, I32, I32, P],
     "pkm_sink_attention": [P, P, P, P, P, I64, P, P, P, P, P, I32, I32, I32, I32, I32, I32, I32, I32, F32, F32, I32,
                            P, P, I32, I32, I32, P],
     "pkm_causal_conv": [P, I32, P, I32, I64, P, P, I32, P, P, P, P, P, P, I32, I32, I32, I32, I32, I32, P],
