@@ -278,6 +278,7 @@ struct PairArgs {
   float* x;
   int W;
   const void* y[2];
+  int f32[2];    // element type of a branch: fp32 (slabs are) or bf16
   int nslab[2];
   int64_t slab_stride;
   const float* w[2];
@@ -289,7 +290,7 @@ struct PairArgs {
 
 // NG >= 1: W % 4 == 0, a thread owns up to NG groups of four coordinates of both branches in registers;
 // NG = 0: any W, one coordinate at a time through LDS.
-template <typename T, typename Y, int NG>
+template <typename T, int NG>
 __global__ void __launch_bounds__(1024) pair_step_kernel(PairArgs a) {
   __shared__ float red[16];
   extern __shared__ __attribute__((aligned(16))) float vbuf[];  // [2][W] (NG = 0)
@@ -304,13 +305,14 @@ __global__ void __launch_bounds__(1024) pair_step_kernel(PairArgs a) {
     float ss[2] = {0.f, 0.f};
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
-      const Y* y = static_cast<const Y*>(a.y[b]) + r * W;
+      const float* yf = static_cast<const float*>(a.y[b]) + r * W;
+      const bf16_t* yh = static_cast<const bf16_t*>(a.y[b]) + r * W;
 #pragma unroll
       for (int it = 0; it < N; ++it) {
         const int i = 4 * (threadIdx.x + it * blockDim.x);
         if (i >= W) break;
-        float4 u = ld4<Y>(y + i);
-        for (int sl = 1; sl < a.nslab[b]; ++sl) u = fma4(1.f, ld4<Y>(y + sl * a.slab_stride + i), u);
+        float4 u = a.f32[b] ? ld4<float>(yf + i) : ld4<bf16_t>(yh + i);
+        for (int sl = 1; sl < a.nslab[b]; ++sl) u = fma4(1.f, ld4<float>(yf + sl * a.slab_stride + i), u);
         v[b][it] = u;
         ss[b] += (u.x * u.x + u.y * u.y) + (u.z * u.z + u.w * u.w);
       }
@@ -340,10 +342,11 @@ __global__ void __launch_bounds__(1024) pair_step_kernel(PairArgs a) {
   }
   float ss[2] = {0.f, 0.f};
   for (int b = 0; b < 2; ++b) {
-    const Y* y = static_cast<const Y*>(a.y[b]) + r * W;
+    const float* yf = static_cast<const float*>(a.y[b]) + r * W;
+    const bf16_t* yh = static_cast<const bf16_t*>(a.y[b]) + r * W;
     for (int i = threadIdx.x; i < W; i += blockDim.x) {
-      float u = ld<Y>(y + i);
-      for (int sl = 1; sl < a.nslab[b]; ++sl) u += ld<Y>(y + sl * a.slab_stride + i);
+      float u = a.f32[b] ? yf[i] : ld<bf16_t>(yh + i);
+      for (int sl = 1; sl < a.nslab[b]; ++sl) u += yf[sl * a.slab_stride + i];
       vbuf[b * W + i] = u;  // read back by this thread only
       ss[b] += u * u;
     }
@@ -490,38 +493,27 @@ PK_EXPORT int pkm_hyper_step(void* xs, int R, int S, int W, const void* y, int y
   return PK_CHECK_LAUNCH();
 }
 
-// x [R, W] fp32, updated in place; ya / yb: [R, W] rows (nslab > 1: fp32 slabs [nslab][R][W]) of one element type; wa, wb,
+// x [R, W] fp32, updated in place; ya / yb: [R, W] rows (na, nb > 1: fp32 slabs [n][R][W]), each of its own element type; wa, wb,
 // post_w [W] fp32; act [R, W] of type act_dt takes the new rows
 PK_EXPORT int pkm_pair_step(void* x, int R, int W, const void* ya, int na, int ya_dt, const void* yb, int nb, int yb_dt,
                             const void* wa, const void* wb, float ca, float cb, const void* post_w, float eps, void* act,
                             int act_dt, hipStream_t stream) {
   if (R <= 0) return 0;
-  if (W < 1 || W > 16384 || na < 1 || nb < 1 || !ya || !yb || !wa || !wb || !post_w || !act || ya_dt != yb_dt) return -1;
-  if (ya_dt != kF32 && (ya_dt != kBF16 || na > 1 || nb > 1)) return -2;
-  const PairArgs a{static_cast<float*>(x), W, {ya, yb}, {na, nb}, static_cast<int64_t>(R) * W,
+  if (W < 1 || W > 16384 || na < 1 || nb < 1 || !ya || !yb || !wa || !wb || !post_w || !act) return -1;
+  if ((ya_dt != kF32 && (ya_dt != kBF16 || na > 1)) || (yb_dt != kF32 && (yb_dt != kBF16 || nb > 1))) return -2;
+  const PairArgs a{static_cast<float*>(x), W, {ya, yb}, {ya_dt == kF32, yb_dt == kF32}, {na, nb}, static_cast<int64_t>(R) * W,
                    {static_cast<const float*>(wa), static_cast<const float*>(wb)}, {ca, cb}, static_cast<const float*>(post_w), eps, act};
-#define PKM_PS(NG, THREADS, LDS)                                                                    \
-  if (ya_dt == kF32) {                                                                              \
-    PKM_DISPATCH(act_dt, E, pair_step_kernel<E, float, NG><<<R, THREADS, LDS, stream>>>(a));        \
-  } else {                                                                                          \
-    PKM_DISPATCH(act_dt, E, pair_step_kernel<E, bf16_t, NG><<<R, THREADS, LDS, stream>>>(a));       \
-  }
+#define PKM_PS(NG, THREADS, LDS) PKM_DISPATCH(act_dt, E, pair_step_kernel<E, NG><<<R, THREADS, LDS, stream>>>(a))
   if (W % 4) {
     const size_t lds = 2 * static_cast<size_t>(W) * sizeof(float);
     const int threads = W >= 4096 ? 1024 : 256;
     if (lds > 60 * 1024) {
-      const void* kern = nullptr;
-      if (ya_dt == kF32) {
-        kern = act_dt == kF32 ? reinterpret_cast<const void*>(pair_step_kernel<float, float, 0>)
-                              : reinterpret_cast<const void*>(pair_step_kernel<bf16_t, float, 0>);
-      } else {
-        kern = act_dt == kF32 ? reinterpret_cast<const void*>(pair_step_kernel<float, bf16_t, 0>)
-                              : reinterpret_cast<const void*>(pair_step_kernel<bf16_t, bf16_t, 0>);
-      }
+      const void* kern = act_dt == kF32 ? reinterpret_cast<const void*>(pair_step_kernel<float, 0>)
+                                        : reinterpret_cast<const void*>(pair_step_kernel<bf16_t, 0>);
       const hipError_t e = hipFuncSetAttribute(kern, hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds));
       if (e != hipSuccess) return static_cast<int>(e);
     }
-    PKM_PS(0, threads, lds)
+    PKM_PS(0, threads, lds);
     return PK_CHECK_LAUNCH();
   }
   // prompt-sized launches: up to four groups per thread (few waves per token, many tokens per CU); decode-sized
@@ -531,11 +523,11 @@ PK_EXPORT int pkm_pair_step(void* x, int R, int W, const void* ya, int na, int y
   threads = threads > 1024 ? 1024 : threads;
   const int per = (groups + threads - 1) / threads;
   if (per <= 1) {
-    PKM_PS(1, threads, 0)
+    PKM_PS(1, threads, 0);
   } else if (per <= 2) {
-    PKM_PS(2, threads, 0)
+    PKM_PS(2, threads, 0);
   } else {
-    PKM_PS(4, threads, 0)
+    PKM_PS(4, threads, 0);
   }
 #undef PKM_PS
   return PK_CHECK_LAUNCH();

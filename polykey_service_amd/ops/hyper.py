@@ -100,7 +100,7 @@ def pair_step(x: torch.Tensor, ya, yb, wa: torch.Tensor, wb: torch.Tensor, ca: f
 
         y = ca U(ya) wa + cb U(yb) wb        x <- x + U(y) post_w        U(u) = u / sqrt(mean(u^2) + eps)
 
-    ``ya``, ``yb``: [T, W] tensors of one element type, or the decode GEMM's unreduced split-K slabs.  Returns
+    ``ya``, ``yb``: [T, W] tensors, or the decode GEMM's unreduced split-K slabs, each as it comes.  Returns
     x in ``act_dtype`` (the next sublayer's input)."""
     T, S, W = x.shape
     assert S == 1 and x.dtype == torch.float32 and x.is_contiguous()
