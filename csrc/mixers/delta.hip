@@ -89,6 +89,104 @@ conv_unit_kernel(float* __restrict__ out, const T* __restrict__ proj, int64_t st
   for (int d = lane; d < width; d += 64) out[static_cast<int64_t>(t) * C + c0 + d] *= k;  // the lane's own values
 }
 
+// Prompt portions in bf16: a thread owns 8 channels (16-byte accesses) of a run of kRunT tokens, win[j] is
+// the input of K - 1 - j tokens ago, refilled from the portion or the slot where the run or a sequence starts;
+// the lanes of one q / k head (D / 8, a power of two) sum their squares by lane exchanges.  Channels
+// beyond C are the decays'.  The same sums in tap order as above.
+constexpr int kRunT = 8;
+
+template <int K>
+__global__ void __launch_bounds__(256)
+conv_unit_run_kernel(float* __restrict__ out, const bf16_t* __restrict__ proj, int64_t stride, const float* __restrict__ taps,
+                     const float* __restrict__ conv_state, const int* __restrict__ cu_q, const int* __restrict__ positions,
+                     const int* __restrict__ slots, const int* __restrict__ token_seq, int T, int G, int D, int H, int V,
+                     ChannelDecay cd) {
+  const int C = 2 * G * D + H * V;
+  int c = 8 * (blockIdx.y * 256 + threadIdx.x);
+  const int t0 = blockIdx.x * kRunT, t1 = min(T, t0 + kRunT);
+  if (c >= C) {
+    c -= C;
+    if (!cd.gates || c >= H * D) return;
+    const float rate = -expf(cd.a_log[c / D]);
+    float bias[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) bias[e] = cd.dt_bias[c + e];
+    pk::u32x4 raw[kRunT];
+#pragma unroll
+    for (int i = 0; i < kRunT; ++i)
+      if (t0 + i < t1) raw[i] = *reinterpret_cast<const pk::u32x4*>(static_cast<const bf16_t*>(cd.z) + (t0 + i) * cd.stride + c);
+#pragma unroll
+    for (int i = 0; i < kRunT; ++i) {
+      if (t0 + i >= t1) break;
+      float z[8];
+      pk::unpack8(raw[i], z);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) z[e] = expf(rate * softplusf(z[e] + bias[e]));
+      store8(cd.gates + static_cast<int64_t>(t0 + i) * H * D + c, z);
+    }
+    return;
+  }
+  const bool qk = c < 2 * G * D;
+  const float post = c < G * D ? 1.f / sqrtf(static_cast<float>(D)) : 1.f;
+  pk::u32x4 raw[kRunT];  // the run's rows, all in flight at once
+#pragma unroll
+  for (int i = 0; i < kRunT; ++i)
+    if (t0 + i < t1) raw[i] = *reinterpret_cast<const pk::u32x4*>(proj + (t0 + i) * stride + c);
+  float w[8][K], win[K][8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e)
+#pragma unroll
+    for (int j = 0; j < K; ++j) w[e][j] = taps[static_cast<int64_t>(c + e) * K + j];
+  int s = token_seq[t0], q0 = cu_q[s];
+  const bool one = s == token_seq[t1 - 1];  // the run lies in one sequence
+#pragma unroll
+  for (int r = 0; r < kRunT; ++r) {
+    const int t = t0 + r;
+    if (t >= t1) break;
+    if (!one) {
+      s = token_seq[t];
+      q0 = cu_q[s];
+    }
+    const int i = t - q0;
+    if (r == 0 || i == 0) {
+      const int slot = slots[s];
+      const bool carry = slot >= 0 && positions[q0] > 0;
+#pragma unroll
+      for (int j = 0; j < K - 1; ++j) {  // win[j + 1] moves to win[j] below
+        const int src = i - (K - 1) + j;
+        if (src >= 0) {
+          load8(proj + (q0 + src) * stride + c, win[j + 1]);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            win[j + 1][e] = carry ? conv_state[(static_cast<int64_t>(slot) * (K - 1) + (K - 1 + src)) * C + c + e] : 0.f;
+        }
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < K - 1; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) win[j][e] = win[j + 1][e];
+    pk::unpack8(raw[r], win[K - 1]);
+    float y[8], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float acc = 0.f;
+#pragma unroll
+      for (int j = 0; j < K; ++j) acc += w[e][j] * win[j][e];
+      y[e] = siluf(acc);
+      ss += y[e] * y[e];
+    }
+    if (qk) {
+      for (int o = D / 16; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+      const float k = post / sqrtf(ss + 1e-6f);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y[e] *= k;
+    }
+    store8(out + static_cast<int64_t>(t) * C + c, y);
+  }
+}
+
 // new state[j] = the input K - 1 - j steps before the portion's end; thread per (sequence, channel)
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -279,6 +377,31 @@ PK_EXPORT int pkm_conv_unit(void* out, const void* proj, long long stride, const
   if (single && n_seqs != T) return -1;
   const int C = 2 * G * D + H * V;
   const ChannelDecay cd{static_cast<float*>(gates), z, z_stride, static_cast<const float*>(a_log), static_cast<const float*>(dt_bias)};
+  const bool runs = !single && T >= 64 && K >= 2 && K <= 4 && dt == kBF16 && D % 8 == 0 && D <= 512 && ((D / 8) & (D / 8 - 1)) == 0 &&
+                    V % 8 == 0 && stride % 8 == 0 && aligned16(proj) && aligned16(out) &&
+                    (!gates || (z_stride % 8 == 0 && aligned16(z) && aligned16(gates)));
+  if (runs) {
+    const dim3 rgrid((T + kRunT - 1) / kRunT, ((C + (gates ? H * D : 0)) / 8 + 255) / 256);
+#define PKM_CU(KK)                                                                                                       \
+  conv_unit_run_kernel<KK><<<rgrid, 256, 0, stream>>>(                                                                   \
+      static_cast<float*>(out), static_cast<const bf16_t*>(proj), stride, static_cast<const float*>(taps),               \
+      static_cast<const float*>(conv_state), static_cast<const int*>(cu_q), static_cast<const int*>(positions),          \
+      static_cast<const int*>(slots), static_cast<const int*>(token_seq), T, G, D, H, V, cd)
+    if (K == 2) {
+      PKM_CU(2);
+    } else if (K == 3) {
+      PKM_CU(3);
+    } else {
+      PKM_CU(4);
+    }
+#undef PKM_CU
+    const int rc = PK_CHECK_LAUNCH();
+    if (rc) return rc;
+    conv_state_kernel<bf16_t><<<dim3((C + 255) / 256, n_seqs), 256, 0, stream>>>(
+        static_cast<float*>(conv_state), static_cast<const bf16_t*>(proj), stride, K, static_cast<const int*>(cu_q),
+        static_cast<const int*>(positions), static_cast<const int*>(slots), C);
+    return PK_CHECK_LAUNCH();
+  }
   const dim3 grid(T, 2 * G + H + (gates ? H : 0));
   PKM_DISPATCH(dt, E, conv_unit_kernel<E><<<grid, 64, 0, stream>>>(
                           static_cast<float*>(out), static_cast<const E*>(proj), stride, static_cast<const float*>(taps), K,

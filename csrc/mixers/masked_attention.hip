@@ -105,6 +105,84 @@ rotate_cache_kernel(T* __restrict__ q_out, const T* __restrict__ proj, int64_t s
   }
 }
 
+struct RotateArgs {
+  void* q_out;
+  const void* proj;
+  int64_t stride;
+  const int* positions;
+  const int* slot_mapping;
+  const float* table;
+  int pairs, table_rows;
+  void* k_cache;
+  void* v_cache;
+  int QH, KH, VH, D, V, bs;
+  const float* q_norm;
+  const float* k_norm;
+  float eps, temp_coef;
+  int temp_every;
+};
+
+// The same with 8 coordinates per thread (16-byte accesses): D and V multiples of 8, D / 8 a power of two up to
+// 64 (the lanes of a head sum their squares by exchanges), pairs a multiple of 8 in the halves layout, plain
+// values.  The partner coordinates of a turned pair are read again (first-level cache).
+template <typename T>
+__global__ void __launch_bounds__(256) rotate_cache_vec_kernel(RotateArgs a) {
+  const int64_t t = blockIdx.y;
+  const int D = a.D, V = a.V, c = 8 * (blockIdx.x * 256 + threadIdx.x);
+  const int nq = a.QH * D, nk = a.KH * D;
+  if (c >= nq + nk + a.VH * V) return;
+  const T* row = static_cast<const T*>(a.proj) + t * a.stride;
+  const int slot = a.slot_mapping[t];
+  float x[8];
+  load8(row + c, x);
+  if (c >= nq + nk) {
+    if (slot < 0) return;
+    const int cv = c - nq - nk, g = cv / V;
+    store8(static_cast<T*>(a.v_cache) + ((static_cast<int64_t>(slot / a.bs) * a.VH + g) * a.bs + slot % a.bs) * V + (cv - g * V), x);
+    return;
+  }
+  const bool query = c < nq;
+  const int ck = query ? c : c - nq, h = ck / D, d = ck - h * D;
+  const float* nw = query ? a.q_norm : a.k_norm;
+  float k = 1.f;
+  const int pos = max(a.positions[t], 0);
+  if (query && a.temp_every > 0) k = 1.f + a.temp_coef * logf(static_cast<float>((pos + 1) / a.temp_every + 1));
+  if (nw) {
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+    for (int o = D / 16; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    k /= sqrtf(ss / static_cast<float>(D) + a.eps);
+  }
+  auto scale = [&](float* v, int at) {
+    float w[8];
+    if (nw) load8(nw + at, w);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= nw ? k * w[e] : k;
+  };
+  scale(x, d);
+  if (a.table && d < 2 * a.pairs) {
+    const bool first = d < a.pairs;
+    const int i = first ? d : d - a.pairs, od = first ? d + a.pairs : i;
+    const float* cs = a.table + (static_cast<int64_t>(clamp_pos(pos, a.table_rows)) * a.pairs + i) * 2;
+    float y[8], t0[8], t1[8];
+    load8(row + (c - d) + od, y);
+    load8(cs, t0);
+    load8(cs + 8, t1);
+    scale(y, od);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float co = e < 4 ? t0[2 * (e & 3)] : t1[2 * (e & 3)], si = e < 4 ? t0[2 * (e & 3) + 1] : t1[2 * (e & 3) + 1];
+      x[e] = first ? x[e] * co - y[e] * si : x[e] * co + y[e] * si;
+    }
+  }
+  if (query) {
+    store8(static_cast<T*>(a.q_out) + t * nq + c, x);
+  } else if (slot >= 0) {
+    store8(static_cast<T*>(a.k_cache) + ((static_cast<int64_t>(slot / a.bs) * a.KH + h) * a.bs + slot % a.bs) * D + d, x);
+  }
+}
+
 // blockIdx.y: 0 the query latent, 1 the key / value latent and the shared key part
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -766,6 +844,46 @@ head_norm_gate_kernel(OT* __restrict__ out, int64_t out_stride, const float* __r
   }
 }
 
+// The same with 8 coordinates per thread: V / 8 a power of two up to 64, 16-byte accesses everywhere.
+template <typename GT, typename OT>
+__global__ void __launch_bounds__(256)
+head_norm_gate_vec_kernel(OT* __restrict__ out, int64_t out_stride, const float* __restrict__ a, int H, int V, float eps,
+                          const GT* __restrict__ gate, int64_t gate_stride, int gate_kind, const float* __restrict__ weight,
+                          int weight_hs, float post, int pair_group, float coef) {
+  const int64_t t = blockIdx.y;
+  const int c = 8 * (blockIdx.x * 256 + threadIdx.x);
+  if (c >= H * V) return;
+  const int h = c / V, d = c - h * V;
+  float u[8];
+  if (pair_group > 0) {
+    const int g = h / pair_group, j = h - g * pair_group;
+    const float* u1 = a + (t * 2 * H + static_cast<int64_t>(g) * 2 * pair_group + j) * V + d;
+    float v[8];
+    load8(u1, u);
+    load8(u1 + static_cast<int64_t>(pair_group) * V, v);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) u[e] -= coef * v[e];
+  } else {
+    load8(a + (t * H + h) * V + d, u);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ss += u[e] * u[e];
+  for (int o = V / 16; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  const float k = post / sqrtf(ss / static_cast<float>(V) + eps);
+  float w[8], g[8];
+  if (weight) load8(weight + static_cast<int64_t>(h) * weight_hs + d, w);
+  if (gate) load8(gate + t * gate_stride + c, g);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    float z = u[e] * k;
+    if (weight) z *= w[e];
+    if (gate) z *= gate_kind == kGateSigmoid ? sigmoidf(g[e]) : g[e] * sigmoidf(g[e]);
+    u[e] = z;
+  }
+  store8(out + t * out_stride + c, u);
+}
+
 }  // namespace
 
 // proj [T, QH*D | KH*D | VH*V] rows `stride` elements apart; table [table_rows, pairs, 2] fp32 or null;
@@ -778,6 +896,16 @@ PK_EXPORT int pkm_rotate_cache(void* q_out, const void* proj, long long stride, 
                                int temp_every, int dt, hipStream_t stream) {
   if (T <= 0) return 0;
   if (D < 1 || V < 1 || 2 * pairs > D || (table && table_rows < 1) || bs < 1 || temp_every < 0) return -1;
+  if (!v_unit && D % 8 == 0 && V % 8 == 0 && D <= 512 && ((D / 8) & (D / 8 - 1)) == 0 && stride % 8 == 0 &&
+      (!table || (halves && pairs % 8 == 0)) && aligned16(q_out) && aligned16(proj) && aligned16(k_cache) && aligned16(v_cache) &&
+      aligned16(q_norm) && aligned16(k_norm) && aligned16(table)) {
+    const RotateArgs a{q_out, proj, stride, static_cast<const int*>(positions), static_cast<const int*>(slot_mapping),
+                       static_cast<const float*>(table), pairs, table_rows, k_cache, v_cache, QH, KH, VH, D, V, bs,
+                       static_cast<const float*>(q_norm), static_cast<const float*>(k_norm), eps, temp_coef, temp_every};
+    const dim3 vgrid((((QH + KH) * D + VH * V) / 8 + 255) / 256, T);
+    PKM_DISPATCH(dt, E, rotate_cache_vec_kernel<E><<<vgrid, 256, 0, stream>>>(a));
+    return PK_CHECK_LAUNCH();
+  }
   const dim3 grid(T, QH + KH + VH);
   PKM_DISPATCH(dt, E, rotate_cache_kernel<E><<<grid, 64, 0, stream>>>(
                           static_cast<E*>(q_out), static_cast<const E*>(proj), stride, static_cast<const int*>(positions),
@@ -916,12 +1044,19 @@ PK_EXPORT int pkm_head_norm_gate(void* out, long long out_stride, const void* a,
   if (T <= 0) return 0;
   if (H < 1 || V < 1 || pair_group < 0 || (pair_group > 0 && H % pair_group) || out_stride < static_cast<long long>(H) * V)
     return -1;
-  const dim3 grid(T, H);
-#define PKM_HNG(GT)                                                                                                  \
-  PKM_DISPATCH(out_dt, O, head_norm_gate_kernel<GT, O><<<grid, 64, 0, stream>>>(                                       \
-                              static_cast<O*>(out), out_stride, static_cast<const float*>(a), H, V, eps,             \
-                              static_cast<const GT*>(gate), gate_stride, gate_kind, static_cast<const float*>(weight),   \
-                              weight_hs, post, pair_group, coef))
+  if (gate_kind == kGateNone) gate = nullptr;
+  const bool vec = V % 8 == 0 && V <= 512 && ((V / 8) & (V / 8 - 1)) == 0 && out_stride % 8 == 0 && aligned16(out) && aligned16(a) &&
+                   aligned16(weight) && (!gate || (gate_stride % 8 == 0 && aligned16(gate)));
+  const dim3 grid(T, H), vgrid((H * V / 8 + 255) / 256, T);
+#define PKM_HNG_ARGS(GT, O)                                                                                                  \
+  static_cast<O*>(out), out_stride, static_cast<const float*>(a), H, V, eps, static_cast<const GT*>(gate), gate_stride,      \
+      gate_kind, static_cast<const float*>(weight), weight_hs, post, pair_group, coef
+#define PKM_HNG(GT)                                                                                                          \
+  if (vec) {                                                                                                                 \
+    PKM_DISPATCH(out_dt, O, head_norm_gate_vec_kernel<GT, O><<<vgrid, 256, 0, stream>>>(PKM_HNG_ARGS(GT, O)));               \
+  } else {                                                                                                                   \
+    PKM_DISPATCH(out_dt, O, head_norm_gate_kernel<GT, O><<<grid, 64, 0, stream>>>(PKM_HNG_ARGS(GT, O)));                     \
+  }
   if (gate_dt == kF32) {
     PKM_HNG(float);
   } else if (gate_dt == kBF16) {
@@ -930,5 +1065,6 @@ PK_EXPORT int pkm_head_norm_gate(void* out, long long out_stride, const void* a,
     return -2;
   }
 #undef PKM_HNG
+#undef PKM_HNG_ARGS
   return PK_CHECK_LAUNCH();
 }

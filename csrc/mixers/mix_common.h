@@ -24,6 +24,20 @@ __device__ __forceinline__ void st<bf16_t>(bf16_t* p, float v) { *p = pk::f2bf(v
 
 __device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z)); }
 
+// 8 consecutive elements at a 16-byte address
+__device__ __forceinline__ void load8(const float* p, float* f) {
+  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+  f[0] = a.x, f[1] = a.y, f[2] = a.z, f[3] = a.w, f[4] = b.x, f[5] = b.y, f[6] = b.z, f[7] = b.w;
+}
+__device__ __forceinline__ void load8(const bf16_t* p, float* f) { pk::unpack8(*reinterpret_cast<const pk::u32x4*>(p), f); }
+__device__ __forceinline__ void store8(float* p, const float* f) {
+  *reinterpret_cast<float4*>(p) = float4{f[0], f[1], f[2], f[3]};
+  *reinterpret_cast<float4*>(p + 4) = float4{f[4], f[5], f[6], f[7]};
+}
+__device__ __forceinline__ void store8(bf16_t* p, const float* f) { *reinterpret_cast<pk::u32x4*>(p) = pk::pack8(f); }
+
+inline bool aligned16(const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; }
+
 // dtype codes of the extern "C" launchers
 constexpr int kBF16 = 0, kF32 = 1;
 

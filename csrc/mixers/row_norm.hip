@@ -17,17 +17,6 @@ namespace {
 
 constexpr int kThreads = 256;
 
-__device__ __forceinline__ void load8(const float* p, float* f) {
-  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
-  f[0] = a.x, f[1] = a.y, f[2] = a.z, f[3] = a.w, f[4] = b.x, f[5] = b.y, f[6] = b.z, f[7] = b.w;
-}
-__device__ __forceinline__ void load8(const bf16_t* p, float* f) { pk::unpack8(*reinterpret_cast<const pk::u32x4*>(p), f); }
-__device__ __forceinline__ void store8(float* p, const float* f) {
-  *reinterpret_cast<float4*>(p) = float4{f[0], f[1], f[2], f[3]};
-  *reinterpret_cast<float4*>(p + 4) = float4{f[4], f[5], f[6], f[7]};
-}
-__device__ __forceinline__ void store8(bf16_t* p, const float* f) { *reinterpret_cast<pk::u32x4*>(p) = pk::pack8(f); }
-
 struct RowArgs {
   void* q_out;
   const void* proj;
@@ -44,81 +33,108 @@ struct RowArgs {
   int QH, KH, D, bs;
 };
 
-// blockIdx.y: 0 the query row, 1 the key row; the biased row waits in LDS for its norm and its partners.
-// VEC: D, the row stride and the base addresses allow 8 elements per access.
-template <typename T, bool VEC>
+// One workgroup per token; the biased row waits in LDS for its two norms and the partners of turned pairs.
+// VEC: D, the row stride and the addresses allow 8 elements per access.  ROT8: and a pair's halves lie whole
+// groups of 8 apart (halves layout, pairs a multiple of 8) or nothing turns.
+template <typename T, bool VEC, bool ROT8>
 __global__ void __launch_bounds__(kThreads) row_norm_cache_kernel(RowArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float row[];  // [heads * D]
+  extern __shared__ __attribute__((aligned(16))) float row[];  // [(QH + KH) * D]
   __shared__ float red[16];
   constexpr int N = VEC ? 8 : 1;
   const int64_t t = blockIdx.x;
-  const bool key = blockIdx.y == 1;
-  const int slot = a.slot_mapping[t], D = a.D;
-  if (key && slot < 0) return;
-  const int n = (key ? a.KH : a.QH) * D, c0 = key ? a.QH * D : 0;
-  const T* src = static_cast<const T*>(a.proj) + t * a.stride + c0;
-  const float* bias = a.bias + c0;
-  const float* w = a.w[key];
-  // element (head h, coordinate d) of the token: q row or cache page
-  const int64_t base = key ? (static_cast<int64_t>(slot / a.bs) * a.KH * a.bs + slot % a.bs) * D : t * n;
-  const int64_t head_stride = key ? static_cast<int64_t>(a.bs) * D : D;
-  T* vdst = static_cast<T*>(a.v_cache);
-  T* dst = static_cast<T*>(key ? a.k_cache : a.q_out);
-  float ss = 0.f;
+  const int slot = a.slot_mapping[t], D = a.D, nq = a.QH * D, n = nq + a.KH * D;
+  const T* src = static_cast<const T*>(a.proj) + t * a.stride;
+  T* q = static_cast<T*>(a.q_out) + t * nq;
+  // head g, coordinate d of the token in a cache: page + g * bs * D + d
+  const int64_t page = slot < 0 ? 0 : (static_cast<int64_t>(slot / a.bs) * a.KH * a.bs + slot % a.bs) * D;
+  T* kc = static_cast<T*>(a.k_cache) + page;
+  T* vc = static_cast<T*>(a.v_cache) + page;
+  const int64_t hs = static_cast<int64_t>(a.bs) * D;
+  float sq = 0.f, sk = 0.f;
   for (int c = N * threadIdx.x; c < n; c += N * kThreads) {
-    float f[N];
+    float f[N], ss = 0.f;
     if constexpr (VEC) {
       float b[8];
       load8(src + c, f);
-      load8(bias + c, b);
+      load8(a.bias + c, b);
 #pragma unroll
       for (int e = 0; e < N; ++e) f[e] += b[e];
+      store8(row + c, f);
     } else {
-      f[0] = ld<T>(src + c) + bias[c];
+      f[0] = ld<T>(src + c) + a.bias[c];
+      row[c] = f[0];
     }
 #pragma unroll
     for (int e = 0; e < N; ++e) ss += f[e] * f[e];
-    if (key) {
-      const int h = c / D;
-      T* v = vdst + base + h * head_stride + (c - h * D);
-      if constexpr (VEC) {
-        store8(v, f);
-      } else {
-        st<T>(v, f[0]);
+    if (c < nq) {
+      sq += ss;
+    } else {
+      sk += ss;
+      if (slot >= 0) {
+        const int h = (c - nq) / D;
+        T* v = vc + h * hs + (c - nq - h * D);
+        if constexpr (VEC) {
+          store8(v, f);
+        } else {
+          st<T>(v, f[0]);
+        }
       }
     }
-    if constexpr (VEC) {
-      store8(row + c, f);
-    } else {
-      row[c] = f[0];
-    }
   }
-  const float k = 1.f / sqrtf(pk::block_sum(ss, red) / static_cast<float>(n) + a.eps);  // (its barriers publish the row)
+  const float kq = 1.f / sqrtf(pk::block_sum(sq, red) / static_cast<float>(nq) + a.eps);  // (the barriers publish the row)
+  const float kk = 1.f / sqrtf(pk::block_sum(sk, red) / static_cast<float>(n - nq) + a.eps);
   int pos = a.positions[t];
   pos = pos < 0 ? 0 : min(pos, a.table_rows - 1);
   const float* cs = a.table ? a.table + static_cast<int64_t>(pos) * a.pairs * 2 : nullptr;
   const int turned = cs ? 2 * a.pairs : 0;
   for (int c = N * threadIdx.x; c < n; c += N * kThreads) {
-    const int h = c / D, d0 = c - h * D;
+    const bool query = c < nq;
+    if (!query && slot < 0) break;
+    const int ck = query ? c : c - nq, h = ck / D, d0 = ck - h * D;
+    const float k = query ? kq : kk;
+    const float* w = query ? a.w[0] : a.w[1] - nq;  // indexed by the row's column
     float f[N];
+    if constexpr (ROT8) {
+      float m[8];
+      load8(row + c, f);
+      load8(w + c, m);
 #pragma unroll
-    for (int e = 0; e < N; ++e) {
-      const int d = d0 + e;
-      float x = row[c + e] * k * w[c + e];
-      if (d < turned) {
-        const bool first = a.halves ? d < a.pairs : (d & 1) == 0;
-        const int i = a.halves ? (first ? d : d - a.pairs) : d >> 1;
-        const int o = c + e + (a.halves ? (first ? a.pairs : -a.pairs) : (first ? 1 : -1));
-        const float y = row[o] * k * w[o];
-        x = first ? x * cs[2 * i] - y * cs[2 * i + 1] : x * cs[2 * i] + y * cs[2 * i + 1];
+      for (int e = 0; e < N; ++e) f[e] *= k * m[e];
+      if (d0 < turned) {
+        const bool first = d0 < a.pairs;
+        const int i = first ? d0 : d0 - a.pairs, o = first ? c + a.pairs : c - a.pairs;
+        float y[8], t0[8], t1[8];
+        load8(row + o, y);
+        load8(w + o, m);
+        load8(cs + 2 * i, t0);
+        load8(cs + 2 * i + 8, t1);
+#pragma unroll
+        for (int e = 0; e < N; ++e) {
+          const float co = e < 4 ? t0[2 * (e & 3)] : t1[2 * (e & 3)], si = e < 4 ? t0[2 * (e & 3) + 1] : t1[2 * (e & 3) + 1];
+          const float p = y[e] * k * m[e];
+          f[e] = first ? f[e] * co - p * si : f[e] * co + p * si;
+        }
       }
-      f[e] = x;
-    }
-    T* o = dst + base + h * head_stride + d0;
-    if constexpr (VEC) {
-      store8(o, f);
     } else {
-      st<T>(o, f[0]);
+#pragma unroll
+      for (int e = 0; e < N; ++e) {
+        const int d = d0 + e;
+        float x = row[c + e] * k * w[c + e];
+        if (d < turned) {
+          const bool first = a.halves ? d < a.pairs : (d & 1) == 0;
+          const int i = a.halves ? (first ? d : d - a.pairs) : d >> 1;
+          const int o = c + e + (a.halves ? (first ? a.pairs : -a.pairs) : (first ? 1 : -1));
+          const float y = row[o] * k * w[o];
+          x = first ? x * cs[2 * i] - y * cs[2 * i + 1] : x * cs[2 * i] + y * cs[2 * i + 1];
+        }
+        f[e] = x;
+      }
+    }
+    T* dst = query ? q + c : kc + h * hs + d0;
+    if constexpr (VEC) {
+      store8(dst, f);
+    } else {
+      st<T>(dst, f[0]);
     }
   }
 }
@@ -176,11 +192,11 @@ int allow_lds(K kern, size_t lds) {
                                               static_cast<int>(lds)));
 }
 
-template <typename T, bool VEC>
+template <typename T, bool VEC, bool ROT8>
 int launch_row(const RowArgs& a, int tokens, size_t lds, hipStream_t stream) {
-  const int rc = allow_lds(row_norm_cache_kernel<T, VEC>, lds);
+  const int rc = allow_lds(row_norm_cache_kernel<T, VEC, ROT8>, lds);
   if (rc) return rc;
-  row_norm_cache_kernel<T, VEC><<<dim3(tokens, 2), kThreads, lds, stream>>>(a);
+  row_norm_cache_kernel<T, VEC, ROT8><<<tokens, kThreads, lds, stream>>>(a);
   return PK_CHECK_LAUNCH();
 }
 
@@ -195,8 +211,6 @@ int launch_group(void* out, const void* y, const void* z, int64_t zs, const void
   return PK_CHECK_LAUNCH();
 }
 
-bool aligned16(const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; }
-
 }  // namespace
 
 // proj [T, QH*D | KH*D] rows `stride` elements apart; bias [(QH + KH) * D], q_w [QH * D], k_w [KH * D] fp32; table
@@ -208,17 +222,20 @@ PK_EXPORT int pkm_row_norm_cache(void* q_out, const void* proj, long long stride
   if (T <= 0) return 0;
   if (D < 1 || QH < 1 || KH < 1 || bs < 1 || 2 * pairs > D || (table && table_rows < 1)) return -1;
   if (!bias || !q_w || !k_w || stride < static_cast<long long>(QH + KH) * D) return -1;
-  const size_t lds = static_cast<size_t>(QH > KH ? QH : KH) * D * sizeof(float);
+  const size_t lds = static_cast<size_t>(QH + KH) * D * sizeof(float);
   if (lds > kMaxLds) return -1;
   const RowArgs a{q_out, proj, stride, static_cast<const float*>(bias), {static_cast<const float*>(q_w), static_cast<const float*>(k_w)},
                   eps, static_cast<const int*>(positions), static_cast<const int*>(slot_mapping), static_cast<const float*>(table),
                   pairs, table_rows, halves, k_cache, v_cache, QH, KH, D, bs};
   const bool vec = D % 8 == 0 && stride % 8 == 0 && aligned16(proj) && aligned16(bias) && aligned16(q_out) && aligned16(k_cache) &&
-                   aligned16(v_cache);
-  if (vec) {
-    PKM_DISPATCH(dt, E, return (launch_row<E, true>(a, T, lds, stream)));
+                   aligned16(v_cache) && aligned16(q_w) && aligned16(k_w);
+  if (vec && (!table || (halves && pairs % 8 == 0 && aligned16(table)))) {
+    PKM_DISPATCH(dt, E, return (launch_row<E, true, true>(a, T, lds, stream)));
   }
-  PKM_DISPATCH(dt, E, return (launch_row<E, false>(a, T, lds, stream)));
+  if (vec) {
+    PKM_DISPATCH(dt, E, return (launch_row<E, true, false>(a, T, lds, stream)));
+  }
+  PKM_DISPATCH(dt, E, return (launch_row<E, false, false>(a, T, lds, stream)));
   return 0;
 }
 

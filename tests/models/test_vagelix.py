@@ -209,18 +209,19 @@ def test_norm_over_all_heads_with_keys_as_values(device, dtype, QH, KH, D, rot, 
 
 
 @pytest.mark.parametrize("device", DEVICES)
-def test_query_temperature_steps_at_its_multiples(device):
+@pytest.mark.parametrize("D,rots", [(10, (6, 4)), (64, (32, 16)), (16, (16, 6)), (8, (0, 0))])
+def test_query_temperature_steps_at_its_multiples(device, D, rots):
     """1 + coef ln(floor((p + 1) / every) + 1): positions around the steps, keys untouched; with and without
-    head norms and a rotation."""
+    head norms and a rotation, at sizes of the scalar and of the 16-byte form."""
     from polykey_service_amd.models.config import RotarySpec
     from polykey_service_amd.ops import masked_attention as ma
-    dev, D, T = torch.device(device), 10, 70
+    dev, T = torch.device(device), 70
     g = torch.Generator().manual_seed(2)
     row = torch.randn(3 * D, generator=g)
     proj = row.repeat(T, 1)
     qn, kn = torch.randn(D, generator=g), torch.randn(D, generator=g)
     pos = torch.arange(T, dtype=torch.int32)
-    for norms, rot in ((True, 0), (False, 0), (True, 6), (False, 4)):
+    for norms, rot in ((True, 0), (False, 0), (True, rots[0]), (False, rots[1])):
         kc, vc = torch.zeros((3, 1, BS, D), device=dev), torch.zeros((3, 1, BS, D), device=dev)
         table = ma.table_for(RotarySpec(rot, 30.0, None, True), T, dev) if rot else None
         kw = dict(q_norm=qn.to(dev), k_norm=kn.to(dev), eps=1e-4) if norms else {}
@@ -230,6 +231,13 @@ def test_query_temperature_steps_at_its_multiples(device):
         f = O.query_temperature(T, 0.7, 16)
         close(got, plain * f.float()[:, None, None], 1e-5)
         assert torch.equal(kc, k0)
+        q, k = row[:D].double().repeat(T, 1)[:, None], row[D:2 * D].double().repeat(T, 1)[:, None]
+        if norms:
+            q, k = O.unit(q, 1e-4) * qn, O.unit(k, 1e-4) * kn
+        close(plain, O.rotate(q, rot, 30.0), 1e-4)
+        at = pos.long()
+        close(kc[at // BS, :, at % BS], O.rotate(k, rot, 30.0), 1e-4)
+        close(vc[at // BS, 0, at % BS], row[2 * D:].repeat(T, 1), 1e-6)
         for p, want in ((0, 0), (14, 0), (15, 1), (30, 1), (31, 2), (62, 3), (63, 4)):
             assert abs(float(f[p]) - (1 + 0.7 * math.log(want + 1))) < 1e-12
 
@@ -334,6 +342,74 @@ def test_filters_unit_vectors_and_decays_in_a_batch(device, G, D, H, V, K):
                 close(state[slots[i]], last, 1e-6)
         close(gates, O.channel_decay(z[:, :H * D].double(), a_log.double(), bias.double()), 1e-4)
     assert float((state[1] - 4).abs().max()) == 0 == float((state[2] - 4).abs().max())
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("G,D,H,V,K", [(2, 64, 4, 128, 4), (1, 8, 3, 16, 2), (3, 128, 3, 24, 3), (1, 512, 1, 8, 4)])
+def test_filters_over_runs_of_tokens_in_a_batch(G, D, H, V, K):
+    """bf16 rows long enough for the run form: several sequences, some short, two continuing from their slots,
+    one without a slot."""
+    from polykey_service_amd.ops import delta as dl
+    dev, C = torch.device("cuda"), 2 * G * D + H * V
+    lens, starts, slots = [3, 70, 1, 2, 41, 8, 16], [0, 5, 40, 0, 0, 7, 0], [4, 2, 7, 0, -1, 5, 3]
+    g = torch.Generator().manual_seed(K + D)
+    T = sum(lens)
+    x, z = torch.randn((T, C + 8), generator=g).bfloat16(), torch.randn((T, H * D + 8), generator=g).bfloat16()
+    taps, a_log, bias = torch.randn((C, K), generator=g), torch.randn(H, generator=g), torch.randn(H * D, generator=g) - 3
+    state = torch.randn((9, K - 1, C), generator=g)
+    cu = [0]
+    for n in lens:
+        cu.append(cu[-1] + n)
+    pos = torch.cat([torch.arange(s, s + n) for s, n in zip(starts, lens)]).int()
+    to = lambda t: t.to(dev)
+    st = to(state)
+    out, gates = dl.conv_unit(to(x)[:, :C], to(taps), st, i32(cu, dev), len(lens), to(pos), i32(slots, dev),
+                              i32(sum([[i] * n for i, n in enumerate(lens)], []), dev), G, D, H, V,
+                              decay=(to(z)[:, 8:8 + H * D], to(a_log), to(bias)))
+    new = state.clone()
+    for i, n in enumerate(lens):
+        past = state[slots[i]].double() if starts[i] and slots[i] >= 0 else torch.zeros((K - 1, C), dtype=D64)
+        xin = torch.cat([past, x[cu[i]:cu[i + 1], :C].double()])
+        y = O.silu(O.causal_filter(xin, taps.double())[K - 1:])
+        qk = y[:, :2 * G * D].view(n, 2 * G, D)
+        qk = qk / torch.sqrt((qk * qk).sum(-1, keepdim=True) + 1e-6)
+        qk[:, :G] /= D ** 0.5
+        close(out[cu[i]:cu[i + 1]], torch.cat([qk.reshape(n, -1), y[:, 2 * G * D:]], 1), 1e-4)
+        if slots[i] >= 0:
+            new[slots[i]] = xin[-(K - 1):].float()
+    close(st, new, 1e-6)
+    close(gates, O.channel_decay(z[:, 8:8 + H * D].double(), a_log.double(), bias.double()), 1e-4)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("H,V", [(4, 64), (6, 8), (2, 512), (3, 24), (5, 7), (2, 128)])
+def test_head_norms_with_every_gate(device, H, V):
+    """One row or the difference of two per head, shared / own / no weights, the three kinds of gates, strided
+    output; sizes of the scalar and of the 16-byte form."""
+    from polykey_service_amd.ops import masked_attention as ma
+    dev, T = torch.device(device), 5
+    g = torch.Generator().manual_seed(V)
+    r = lambda *s: torch.randn(s, generator=g)
+    a, a2, gate = r(T, H, V), r(T, 2 * H, V), r(T, H * V + 8)
+    for kind, act in ((ma.GATE_SIGMOID, O.sigmoid), (ma.GATE_SILU, O.silu), (ma.GATE_NONE, None)):
+        for w in (None, r(V), r(H * V)):
+            for pair in (0, 1, H):
+                u = a.double()
+                if pair:
+                    p5 = a2.double().view(T, H // pair, 2, pair, V)
+                    u = (p5[:, :, 0] - 0.3 * p5[:, :, 1]).reshape(T, H, V)
+                want = O.unit(u, 1e-3) * 0.7
+                if w is not None:
+                    want = want * (w.view(H, V) if w.numel() == H * V else w).double()
+                want = want.reshape(T, H * V)
+                if act is not None:
+                    want = want * act(gate[:, 8:].double())
+                out = torch.zeros((T, H * V + 16), device=dev)
+                ma.head_norm_gate((a2 if pair else a).to(dev), H, V, 1e-3, gate.to(dev)[:, 8:] if act is not None else None, kind,
+                                  torch.float32, weight=None if w is None else w.to(dev), post=0.7, pair_group=pair, coef=0.3,
+                                  out=out[:, 8:8 + H * V])
+                close(out[:, 8:8 + H * V], want, 1e-4)
+                assert float(out[:, :8].abs().max()) == 0 == float(out[:, 8 + H * V:].abs().max())
 
 
 @pytest.mark.parametrize("device", DEVICES)
